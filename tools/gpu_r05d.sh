@@ -1,7 +1,7 @@
 #!/bin/bash
 # Round-5 batch D: A/B of the new batched-decode defaults (resid depth 4, single-matrix depth 2) against
-# further depths, the 256-thread attention, the batch speculative pass; int8 hand-off depth; then the
-# PMC repro bisect (stops at the first crash).
+# further depths, the 256-thread attention, the batch speculative pass; int8 hand-off depth.
+
 set -o pipefail
 R=$GRAFT_REPO_ROOT
 O=$R/gpurun_out/r05d
@@ -22,6 +22,4 @@ chk "ab bs1" $?
 timeout -k 10 300 python -u tools/ab_decode.py --batch 8 --rounds 3 --steps 50 --quantize llm.int8 --variants base \
   di8q3:LIB=scratch/di8q3.so > $O/ab_c3.jsonl 2> $O/ab_c3.err
 chk "ab c3" $?
-PMC_CASES="w4:8:4096:4096 i8q:8:4096:4096 i8q:8:4096:11008 i8swiglu:8:11008:4096 i8:8:4096:4096" bash tools/pmc_repro.sh r05d_pmc_repro
-echo "pmc repro rc=$?" >> $O/status.log
 exit 0

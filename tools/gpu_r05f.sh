@@ -29,6 +29,4 @@ chk "ab bs1" $?
 timeout -k 10 300 python -u tools/ab_decode.py --batch 8 --rounds 3 --steps 50 --quantize llm.int8 --variants base \
   di8q3:LIB=scratch/di8q3.so norm_rowstats:I8_NORM_ROWSTATS=True > $O/ab_c3.jsonl 2> $O/ab_c3.err
 chk "ab c3" $?
-PMC_CASES="w4:8:4096:4096 i8q:8:4096:4096 i8q:8:4096:11008 i8swiglu:8:11008:4096 i8:8:4096:4096" bash tools/pmc_repro.sh r05f_pmc_repro
-echo "pmc repro rc=$?" >> $O/status.log
 exit 0

@@ -17,6 +17,4 @@ timeout -k 10 120 python -u -c "import __graft_entry__ as g; g.smoke()" > $O/smo
 chk "smoke" $?
 timeout -k 10 400 python -u bench.py > $O/bench.json 2> $O/bench.err
 chk "bench" $?
-PMC_CASES="prep:8:4096:4096 qw:4096:4096:4096 gemm_i8:128:4096:4096" bash tools/pmc_repro.sh r05h_pmc_repro
-echo "pmc repro rc=$?" >> $O/status.log
 exit 0
