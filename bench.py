@@ -466,11 +466,12 @@ def cpu_baseline(model, budget_s: float = 20.0):
 
 
 # ----------------------------------------------------------------------------- hybrid models (--hybrid)
-# name -> LLaMA sizes and the Mugivik layers beside them: the same width and depth, sublayer parameters
-# matched (mixers ~4 width^2, feed-forwards equal to the SwiGLU's 3 matrices)
+# name -> LLaMA sizes and the Mugivik and Bobasun layers beside them: the same width and depth, sublayer parameters
+# matched (Mugivik: mixers ~4 width^2, feed-forwards equal to the SwiGLU's 3 matrices; Bobasun: 4 query heads per
+# key / value head, the feed-forward wider by what that saves, 4 residual streams)
 HYBRID_SIZES = {
-    "1B": dict(width=2048, layers=24, heads=16, ff=8448, window=1024),
-    "7B": dict(width=4096, layers=32, heads=32, ff=16512, window=2048),
+    "1B": dict(width=2048, layers=24, heads=16, ff=8448, window=1024, kv_heads=4, glu=6656),
+    "7B": dict(width=4096, layers=32, heads=32, ff=16512, window=2048, kv_heads=8, glu=13056),
 }
 
 
@@ -493,22 +494,30 @@ def hybrid_config(name: str):
     return MugivikConfig(32000, z["width"], 1e-5, 65537, 127, 11, tuple(layers))
 
 
+def bobasun_config(name: str):
+    from lit_llama.bobasun import BobasunConfig, BobasunLayer
+    from lit_llama.mixers import GroupedSpec
+
+    z = HYBRID_SIZES[name]
+    spec = GroupedSpec(z["heads"], z["kv_heads"], 128, 128, 0.1, 128, 10000.0, 2.0, v_mix=True)
+    return BobasunConfig(32000, z["width"], 1e-5, 8.0, 4, tuple(BobasunLayer(spec, z["glu"], 7.0) for _ in range(z["layers"])))
+
+
 def hybrid_leg(name: str, which: str, prompt: int, steps: int, batches=(1, 8)):
     """Prompt tokens/s (one `prompt`-token sequence, every layer and the last row's head, best of 5) and decode
-    tokens/s (graph replays after a 1,000-token prompt) of Mugivik or of the LLaMA of the same size, bf16."""
+    tokens/s (graph replays after a 1,000-token prompt) of Mugivik, Bobasun or the LLaMA of the same size, bf16."""
     import gc
 
-    from lit_llama import LLaMA, LLaMAConfig
+    from lit_llama import Bobasun, LLaMA, LLaMAConfig, Mugivik
     from lit_llama.engine import DecodeSession
-    from lit_llama.mugivik import Mugivik
     from lit_llama.utils import EmptyInitOnDevice
 
     z = HYBRID_SIZES[name]
     g = torch.Generator().manual_seed(5)
-    if which == "mugivik":
-        m = Mugivik.random(hybrid_config(name))
+    if which != "llama":
+        m = Mugivik.random(hybrid_config(name)) if which == "mugivik" else Bobasun.random(bobasun_config(name))
         wb = sum(q.nbytes() for mx in m.mixers for q in mx.linears()) + sum(
-            q.nbytes() for f in m.mlps if f for q in f.linears()) + m.embed.nbytes()
+            q.nbytes() for f in m.mlps if f for q in f.linears()) + m.head.nbytes()
     else:
         cfg = LLaMAConfig(block_size=4096, vocab_size=32000, n_layer=z["layers"], n_head=z["heads"], n_embd=z["width"])
         with EmptyInitOnDevice(device=torch.device("cuda"), dtype=torch.bfloat16):
@@ -618,8 +627,8 @@ def main():
     ap.add_argument("--stub-fail-rank", type=int, default=-1,
                     help="with --stub: this rank exits 3 before the barrier (launcher failure test)")
     ap.add_argument("--hybrid", default=None, metavar="SIZES",
-                    help="instead of the default workload: Mugivik beside LLaMA at these sizes, e.g. 1B,7B (one GPU)")
-    ap.add_argument("--hybrid-models", default="mugivik,llama")
+                    help="instead of the default workload: the hybrid models beside LLaMA at these sizes, e.g. 1B,7B (one GPU)")
+    ap.add_argument("--hybrid-models", default="mugivik,llama", help="of mugivik, bobasun, llama")
     ap.add_argument("--hybrid-batches", default="1,8")
     ap.add_argument("--hybrid-prompt", type=int, default=2048)
     args = ap.parse_args()

@@ -392,8 +392,8 @@ int llj_i8_norm_rowstats(const void* x, const void* norm_w, float eps, void* xn,
 int llj_i8_linear_resid(const void* A, int lda, const void* CB, const void* SCB, void* x, int ldx, int M, int N, int K,
                         const void* stats, void* stream);
 
-/* ---------------------------------------------------------------- hybrid models (post-norm, recurrent, latent)
- * Ops of models outside the LLaMA block (no reference counterpart; lit_llama/mugivik.py). dt: activation
+/* ---------------------------------------------------------------- hybrid models (post-norm, streams, recurrent, latent, grouped-query)
+ * Ops of models outside the LLaMA block (no reference counterpart; lit_llama/mugivik.py, lit_llama/bobasun.py). dt: activation
  * type of every void* operand, 0 bf16 / 1 fp32; residual, norms, scores and recurrent state are fp32.
  * A call's activation rows are either packed prompt rows -- row_seq[m] = sequence of row m, sequence b's
  * rows row0[b] .. row0[b + 1] - 1 -- or, with row_seq (and row0) NULL, one decode row per sequence.
@@ -416,18 +416,24 @@ int llj_post_norm(const void* t, int ldt, const void* w, float eps, float* x, in
                   const int* rows, int M, int C, int dt, void* stream);
 /* h = max(h, 0)^2 in place */
 int llj_g_relu2(void* h, size_t n, int dt, void* stream);
-/* out[m] = A[m] . W^T for M <= 16 bf16 rows, the weight (N, K) read once; act 1: max(., 0)^2. N % 16 == 0,
- * K % 128 == 0. */
-int llj_rows_linear(int act, const void* A, int lda, const void* W, void* out, int ldo, int M, int N, int K, void* stream);
+/* A Linear's bias and activation, act of the products below: 0 none; 1 max(., 0)^2 (without bias); 2 the clamped gated
+ * unit of interleaved columns, gate g at 2 j and up u at 2 j + 1: g' = min(g, limit), u' = clamp(u, -limit, limit),
+ * output column j = g' sigmoid(alpha g') (u' + 1). bias: fp32 (N) or NULL.
+ * llj_g_bias_act, any sizes, after a product: act 0 y += bias in place (out NULL), act 2 out[M, N / 2]. */
+int llj_g_bias_act(int act, void* y, int ldy, const float* bias, void* out, int ldo, int M, int N, float limit, float alpha,
+                   int dt, void* stream);
+/* out[m] = act(A[m] . W^T + bias) for M <= 16 bf16 rows, the weight (N, K) read once. N % 16 == 0, K % 128 == 0. */
+int llj_rows_linear(int act, const void* A, int lda, const void* W, const float* bias, void* out, int ldo, int M, int N, int K,
+                    float limit, float alpha, void* stream);
 /* One bf16 row with llj_post_norm in front: x_out = x + t / rms(t) * (1 + norm_w) (fp32, width C <= K, C % 8
  * == 0, C <= 8192), out = act(bf16(x_out) . W^T). x_out must not be x. */
 int llj_post_linear(int act, const void* t, const void* norm_w, float eps, const float* x, float* x_out, int C,
                     const void* W, void* out, int N, int K, void* stream);
-/* C = act(A . W^T) for many bf16 rows on the prefill GEMM (N, K multiples of 128); ws (act 0, optional,
+/* C = act(A . W^T + bias) for many bf16 rows on the prefill GEMM (N, K multiples of 128); ws (act 0, optional,
  * llj_gemm_bf16_ws_bytes bytes): K split over workgroups when the row tiles leave most CUs idle. */
 size_t llj_gemm_bf16_ws_bytes(int M, int N, int K);
-int llj_gemm_bf16(int act, const void* A, int lda, const void* W, void* C, int ldc, int M, int N, int K, void* ws,
-                  size_t ws_bytes, void* stream);
+int llj_gemm_bf16(int act, const void* A, int lda, const void* W, const float* bias, void* C, int ldc, int M, int N, int K,
+                  float limit, float alpha, void* ws, size_t ws_bytes, void* stream);
 /* Gated linear attention token by token (decode steps, short prompts, any sizes): packed projections
  * [q | k | v | g | a] at columns oq, ok, ov, og, oa of `in`; z = a2 . a + a2b, alpha = sigmoid(z)^inv_tau;
  * S = diag(alpha) S + k v^T, o = S^T (q * qscale); y = o / rms(o) * norm_w * silu(g). state
@@ -481,6 +487,52 @@ int llj_latent_decode(const void* in, int ld, int oq, int og, int okv, const voi
                       const void* turns, const int* pos, const int* slot, void* ring, int W, int win, void* qc, float* part,
                       int nsplit, void* y, int ldy, int M, int heads, int dim, int rot_dim, int vdim, int kv_rank, int krp,
                       int ldc, float eps, float scale, void* stream);
+
+/* Residual of several streams (hyper-connections), x [M][streams][ldx] fp32; layer norm with a weight, no bias.
+ * embed: every stream = embed[tok] * scale, h = layer_norm(sum_s in[s] x_s) * norm_w (in NULL: the plain sum); pos
+ * (decode rows, else NULL) is advanced.
+ * step: x_t <- sum_s mix[s][t] x_s + out[t] y from the old streams, then h of the new ones as above; with `rows` output
+ * row i is of row rows[i] and x stays as it is. */
+int llj_streams_embed(const int* tok, const void* embed, int lde, float scale, int* pos, float* x, int ldx, int streams,
+                      const float* in, const void* norm_w, float eps, void* h, int ldh, int M, int C, int dt, void* stream);
+int llj_streams_step(const void* y, int ldy, const float* out, const float* mix, float* x, int ldx, int streams,
+                     const float* in, const void* norm_w, float eps, void* h, int ldh, const int* rows, int M, int C, int dt,
+                     void* stream);
+/* One bf16 row with llj_streams_step in front: x_out = the new streams (x_out must not be x), out = act(bf16(h) . W^T +
+ * bias). llj_streams_linear_ok: the stream counts and widths it takes. */
+int llj_streams_linear_ok(int streams, int C);
+int llj_streams_linear(int act, const void* y, const float* out_w, const float* mix, const float* x, float* x_out, int ldx,
+                       int streams, const float* in, const void* norm_w, float eps, int C, const void* W, const float* bias,
+                       void* out, int N, int K, float limit, float alpha, void* stream);
+/* Grouped-query attention over per-sequence rows [k of kv_heads heads | v of kv_heads heads] at
+ * cache[slot][position] (W rows of stride ldc per slot). Packed projections in `in`: queries at column oq, keys ok,
+ * values ov, one gate per head at og (-1: none).
+ * prep: rotate-half rotation of the first rot_dims dimensions of queries (in place) and keys (turns[i] = frequency of pair
+ * (i, i + rot_dims / 2) / 2 pi, doubles), with qk_norm both divided by their root mean square over dim; key and value
+ * into the cache. first (row stride ldf): without lam a copy of the values is left there, with lam the values are
+ * (1 - lam) v + lam first.
+ * rows: any sizes; softmax over the row's own and all earlier positions of q . k * scale, with sink one added to the
+ * denominator; y = sum p v * sigmoid(gate).
+ * flash: prompt rows (bf16, MFMA); work = two (first row, rows, sequence) blocks of at most `rows` rows each per entry (the
+ * second's rows 0: none), rows = llj_gqa_flash_rows (0: not these sizes).
+ * decode: one row per sequence (bf16, MFMA), prep included; part [M][heads][nsplit][llj_gqa_part_width(vdim)] fp32 scratch,
+ * nsplit <= 64 key ranges. */
+int llj_gqa_prep(void* in, int ld, int oq, int ok, int ov, const void* turns, int rot_dims, int qk_norm, float eps,
+                 const int* pos, const int* row_seq, const int* slot, void* cache, int W, int ldc, void* first,
+                 const float* lam, int ldf, int M, int heads, int kv_heads, int dim, int vdim, int dt, void* stream);
+int llj_gqa_rows(const void* in, int ld, int oq, int og, const int* pos, const int* row_seq, const int* slot, const void* cache,
+                 int W, int ldc, void* y, int ldy, int M, int heads, int kv_heads, int dim, int vdim, float scale, int sink,
+                 int dt, void* stream);
+int llj_gqa_flash_rows(int dim, int vdim, int long_prompt);
+int llj_gqa_flash(const void* in, int ld, int oq, int og, const int* work, int nwork, int rows, const int* pos, const int* slot,
+                  const void* cache, int W, int ldc, void* y, int ldy, int M, int heads, int kv_heads, int dim, int vdim,
+                  float scale, int sink, void* stream);
+int llj_gqa_decode_ok(int dim, int vdim);
+int llj_gqa_part_width(int vdim);
+int llj_gqa_decode(const void* in, int ld, int oq, int ok, int ov, int og, const void* turns, int rot_dims, int qk_norm,
+                   float eps, const int* pos, const int* slot, void* cache, int W, int ldc, void* first, const float* lam,
+                   int ldf, float* part, int nsplit, void* y, int ldy, int M, int heads, int kv_heads, int dim, int vdim,
+                   float scale, int sink, void* stream);
 
 /* Measurement aid (no reference counterpart): reads `bytes` (a multiple of 16) at p once with
  * non-temporal 16-byte loads over `grid` workgroups of 256 and writes one float per workgroup to

@@ -44,6 +44,13 @@ __device__ __forceinline__ void st8(float* p, const float (&v)[8]) {
   reinterpret_cast<float4*>(p)[1] = make_float4(v[4], v[5], v[6], v[7]);
 }
 
+// clamped gated unit: g * sigmoid(alpha g) * (u + 1), g = min(g, limit), u = clamp(u, -limit, limit)
+__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.f + expf(-alpha * g)) * (u + 1.f);
+}
+
 }  // namespace llj
 
 #define LLJ_DT(dt, CALL_BF16, CALL_F32) \

@@ -44,6 +44,7 @@
 #include <cstdlib>
 
 #include "common.h"
+#include "elem.h"
 #include "i8ws.h"
 #include "lit_llama_amd.h"
 
@@ -52,13 +53,17 @@ namespace llj {
 // GWF_W4Z: int4 W4P with integral zeros (LLJ_WF_ZINT) in the convert-once LDS-DMA GEMM (internal)
 enum : int { GWF_W4 = 0, GWF_BF16 = 1, GWF_I8 = 2, GWF_W8 = 3, GWF_W4G = 4, GWF_W4Z = 5 };
 // GEP_RELU2: max(y, 0)^2 (bf16 weights)
+// GEP_BIAS: y + bias[n] (bf16 weights)
+// GEP_GLU: the clamped gated unit (elem.h) of interleaved columns, gate n = 2 j and up n = 2 j + 1 with their bias,
+// into column j of C (bf16 weights)
 // GEP_SWIGLU: h = bf16(silu(bf16(A . W1^T))) * bf16(A . W2^T) in one pass (convert-once int4: both weights'
 // codes staged per chunk, one A tile feeding both; W2 / sz2)
 // GEP_PARTIAL: split-K slice of a residual GEMM -- fp32 partials y (scale applied) of K range slice
 // blockIdx.x % nsplit into ws[slice][M][N]; llj_gemm_resid_ws's reduce adds them and the residual
 // GEP_SWIGLU_PART: split-K slice of the dual SwiGLU pass (its last partial wave of tiles) -- fp32 partials of
 // c_fc1 and c_fc2 (scales applied) into ws[slice][2][M][N]; llj_gemm_swiglu_ws's reduce finishes h
-enum : int { GEP_STORE = 0, GEP_RESID = 1, GEP_QKV = 2, GEP_SILU_MUL = 3, GEP_SWIGLU = 4, GEP_PARTIAL = 5, GEP_SWIGLU_PART = 6, GEP_RELU2 = 7 };
+enum : int { GEP_STORE = 0, GEP_RESID = 1, GEP_QKV = 2, GEP_SILU_MUL = 3, GEP_SWIGLU = 4, GEP_PARTIAL = 5, GEP_SWIGLU_PART = 6, GEP_RELU2 = 7,
+               GEP_BIAS = 8, GEP_GLU = 9 };
 
 struct GemmParams {
   const bf16_t* A;  // (M, K) rows with stride lda
@@ -90,6 +95,9 @@ struct GemmParams {
   // GEP_PARTIAL: nsplit K slices of kcs 64-deep chunks each (kcs even), fp32 partials [nsplit][M][N]
   float* ws;
   int nsplit, kcs;
+  // GEP_BIAS / GEP_GLU: fp32 bias (N) or NULL, the unit's constants
+  const float* bias;
+  float limit, alpha;
 };
 
 // Tile epilogues run in two phases per 16-column block: every element's operand is loaded first
@@ -178,6 +186,11 @@ __device__ __forceinline__ void gemm_store_elem(const GemmParams& p, float y, in
       }
       *reinterpret_cast<uint32_t*>(dst + ei) = ob | (pr << 16);
     }
+  } else if constexpr (EP == GEP_GLU) {  // y: bias added; lanes 0, 1 of a quad hold unit j, lanes 2, 3 unit j + 1
+    const float u = lane_xor1(y);
+    const uint32_t ob = (uint32_t)f2bf(clamped_glu(y, u, p.limit, p.alpha));  // (odd lanes: unused)
+    const uint32_t pr = dpp_u32<kDppXor2>(ob);
+    if (live && !(row & 3)) *reinterpret_cast<uint32_t*>(p.C + (size_t)m * p.ldc + (n >> 1)) = ob | (pr << 16);
   } else {
     bf16_t* cp = p.C + (size_t)(live ? m : M - 1) * p.ldc + n;
     float o;
@@ -628,6 +641,8 @@ __global__ __launch_bounds__(2 * BM) void gemm_kernel(GemmParams p) {
     float2 szn = make_float2(1.f, 0.f);
     if constexpr (NIB) szn = p.sz[n];
     if constexpr (I8) szn.x = reinterpret_cast<const float*>(p.sz)[n];  // SCB
+    float bn = 0.f;
+    if constexpr (EP == GEP_BIAS || EP == GEP_GLU) bn = p.bias ? p.bias[n] : 0.f;
     const int nblk = n0 + wc * 16 * NJ + 16 * j;  // first column of this 16-column block
     const QkvCol qc = EP == GEP_QKV ? qkv_col(p, nblk, n, Cd) : QkvCol{};
     constexpr int GI = I8 ? (EP == GEP_QKV ? 1 : 2) : 4;  // row blocks whose operands are in flight together (LLM.int8: 3 accumulator sets live)
@@ -649,6 +664,7 @@ __global__ __launch_bounds__(2 * BM) void gemm_kernel(GemmParams p) {
           const int m = m0 + ml;
           float y = acc[i0 + i][j][r];
           if constexpr (NIB) y = szn.x * (y - szn.y * rs_lds[ml]);
+          if constexpr (EP == GEP_BIAS || EP == GEP_GLU) y += bn;
           const bool live = m < M;
           if constexpr (I8) {  // mm_dequant in fp16, + the fp16 outlier product, in fp16 (the GEMV's epilogue)
             const float sa = L8.sca[live ? m : M - 1];
@@ -1179,12 +1195,14 @@ __global__ __launch_bounds__(512, 1) void gemm_glds_kernel(GemmParams p) {
     return;
   }
   if constexpr (LLJ_GLDS_LDS_EPI && !NIB && !PART && BN == 128 && MI <= 4 &&
-                (EP == GEP_STORE || EP == GEP_RESID || EP == GEP_SILU_MUL || EP == GEP_SWIGLU || EP == GEP_RELU2))
+                (EP == GEP_STORE || EP == GEP_RESID || EP == GEP_SILU_MUL || EP == GEP_SWIGLU || EP == GEP_RELU2 ||
+                 EP == GEP_BIAS || EP == GEP_GLU))
     if ((p.ldc & 7) == 0 && (reinterpret_cast<uintptr_t>(p.C) & 15) == 0) {
       // the other bf16 epilogues through LDS as well: the tile's bf16 values (y, or the whole SwiGLU product) to
       // LDS in the accumulator layout, then 16-byte row segments (8 columns) per thread, the residual / c_fc1
       // operand read the same way -- rows of 256 (SwiGLU: 128) contiguous bytes instead of 4-byte pairs
-      constexpr int TW = DUAL ? BN / 2 : BN, TP = TW + 8, SEGS = TW / 8, RPP = 512 / SEGS;
+      constexpr bool GLU = EP == GEP_GLU;
+      constexpr int TW = DUAL || GLU ? BN / 2 : BN, TP = TW + 8, SEGS = TW / 8, RPP = 512 / SEGS;
       bf16_t* Ts = reinterpret_cast<bf16_t*>(smem);
       asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
       __syncthreads();  // every wave is past its last fragment read of the K loop
@@ -1192,8 +1210,9 @@ __global__ __launch_bounds__(512, 1) void gemm_glds_kernel(GemmParams p) {
       for (int j = 0; j < (DUAL ? NJ / 2 : NJ); ++j) {
         const int nl = wc * 16 * (DUAL ? NJ / 2 : NJ) + 16 * j + row;
         const float s1 = CVT ? p.sz[n0 + nl].x : 1.f;
-        float s2 = 1.f;
+        float s2 = 1.f, bn = 0.f;
         if constexpr (DUAL) s2 = p.sz2[n0 + nl].x;
+        if constexpr (EP == GEP_BIAS || GLU) bn = p.bias ? p.bias[n0 + nl] : 0.f;
 #pragma unroll
         for (int i = 0; i < MI; ++i)
 #pragma unroll
@@ -1206,8 +1225,15 @@ __global__ __launch_bounds__(512, 1) void gemm_glds_kernel(GemmParams p) {
             } else {
               o = s1 * acc[i][j][r];
               if constexpr (EP == GEP_RELU2) o = fmaxf(o, 0.f) * fmaxf(o, 0.f);
+              if constexpr (EP == GEP_BIAS || GLU) o += bn;
             }
-            Ts[(wr * 16 * MI + 16 * i + 4 * g + r) * TP + nl] = f2bf(o);
+            const int tr = (wr * 16 * MI + 16 * i + 4 * g + r) * TP;
+            if constexpr (GLU) {
+              o = clamped_glu(o, lane_xor1(o), p.limit, p.alpha);
+              if (!(row & 1)) Ts[tr + (nl >> 1)] = f2bf(o);
+            } else {
+              Ts[tr + nl] = f2bf(o);
+            }
           }
       }
       __syncthreads();
@@ -1217,7 +1243,7 @@ __global__ __launch_bounds__(512, 1) void gemm_glds_kernel(GemmParams p) {
         const int rl = tid / SEGS + RPP * k, m = m0 + rl;
         if (m >= M) continue;
         const uint4 v = *reinterpret_cast<const uint4*>(Ts + rl * TP + 8 * seg);
-        uint4* cp = reinterpret_cast<uint4*>(p.C + (size_t)m * p.ldc + n0 + 8 * seg);
+        uint4* cp = reinterpret_cast<uint4*>(p.C + (size_t)m * p.ldc + (GLU ? n0 / 2 : n0) + 8 * seg);
         uint4 o = v;
         if constexpr (EP == GEP_RESID || EP == GEP_SILU_MUL) {
           const uint4 c = *cp;
@@ -1321,6 +1347,8 @@ __global__ __launch_bounds__(512, 1) void gemm_glds_kernel(GemmParams p) {
     const int n = nblk + row;
     float2 szn = make_float2(1.f, 0.f);
     if constexpr (NIB || CVT) szn = p.sz[n];
+    float bn = 0.f;
+    if constexpr (EP == GEP_BIAS || EP == GEP_GLU) bn = p.bias ? p.bias[n] : 0.f;
     const QkvCol qc = EP == GEP_QKV ? qkv_col(p, nblk, n, Cd) : QkvCol{};
     constexpr int GI = EP == GEP_QKV ? (MI > 4 ? 1 : LLJ_QKV_GI) : 4;  // row blocks whose operands are in flight together
 #pragma unroll
@@ -1345,6 +1373,7 @@ __global__ __launch_bounds__(512, 1) void gemm_glds_kernel(GemmParams p) {
           float y = acc[i0 + i][j][r];
           if constexpr (NIB) y = szn.x * (y - szn.y * rs_lds[ml]);
           if constexpr (CVT) y = szn.x * y;
+          if constexpr (EP == GEP_BIAS || EP == GEP_GLU) y += bn;
           gemm_store_elem<EP>(p, y, m, n, m < M, row, Cd, opv[i][r], qg[i][r], qc);
         }
       }

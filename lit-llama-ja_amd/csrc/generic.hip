@@ -94,6 +94,26 @@ __global__ __launch_bounds__(256) void g_linear_kernel(const T* __restrict__ x, 
   }
 }
 
+// ---- a biased Linear's second pass: y += bias in place (act 0), or the clamped gated unit of its interleaved
+// columns (gate 2 j, up 2 j + 1, bias added to both) into out[j] (act 2)
+template <typename T>
+__global__ __launch_bounds__(256) void g_bias_act_kernel(int act, T* y, int ldy, const float* __restrict__ bias, T* out, int ldo,
+                                                         int M, int N, float limit, float alpha) {
+  const int cols = act ? N / 2 : N;
+  const size_t n = (size_t)M * cols;
+  for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (size_t)gridDim.x * 256) {
+    const size_t m = i / cols;
+    const int c = (int)(i - m * cols);
+    if (act) {
+      const float g = ldv(y, m * ldy + 2 * c) + (bias ? bias[2 * c] : 0.f);
+      const float u = ldv(y, m * ldy + 2 * c + 1) + (bias ? bias[2 * c + 1] : 0.f);
+      stv(out, m * ldo + c, clamped_glu(g, u, limit, alpha));
+    } else {
+      stv(y, m * ldy + c, ldv(y, m * ldy + c) + bias[c]);
+    }
+  }
+}
+
 // ---- q / k / v split of c_attn's output (model.py:204), apply_rope on q and k in fp32
 // (model.py:312-329), k / v of the token at position p into cache slot p % S. Block (row, head).
 template <typename TT>
@@ -346,6 +366,19 @@ int llj_g_silu_mul(const void* a1, const void* a2, void* h, size_t n, int dt, vo
   hipStream_t s = (hipStream_t)stream;
   LLJ_DT(dt, hipLaunchKernelGGL(g_silu_mul_kernel<bf16_t>, dim3(g), dim3(256), 0, s, (const bf16_t*)a1, (const bf16_t*)a2, (bf16_t*)h, n),
          hipLaunchKernelGGL(g_silu_mul_kernel<float>, dim3(g), dim3(256), 0, s, (const float*)a1, (const float*)a2, (float*)h, n));
+  LLJ_CHECK_LAUNCH();
+  return 0;
+}
+
+int llj_g_bias_act(int act, void* y, int ldy, const float* bias, void* out, int ldo, int M, int N, float limit, float alpha,
+                   int dt, void* stream) {
+  LLJ_REQUIRE((act == 0 || act == 2) && y && M > 0 && N > 0 && ldy >= N && (dt == 0 || dt == 1));
+  LLJ_REQUIRE(act == 0 ? bias && !out : out && out != y && N % 2 == 0 && ldo >= N / 2);
+  const size_t n = (size_t)M * (act ? N / 2 : N), blocks = (n + 255) / 256;
+  const unsigned g = blocks < 4096 ? (unsigned)blocks : 4096u;
+  hipStream_t s = (hipStream_t)stream;
+  LLJ_DT(dt, hipLaunchKernelGGL(g_bias_act_kernel<bf16_t>, dim3(g), dim3(256), 0, s, act, (bf16_t*)y, ldy, bias, (bf16_t*)out, ldo, M, N, limit, alpha),
+         hipLaunchKernelGGL(g_bias_act_kernel<float>, dim3(g), dim3(256), 0, s, act, (float*)y, ldy, bias, (float*)out, ldo, M, N, limit, alpha));
   LLJ_CHECK_LAUNCH();
   return 0;
 }

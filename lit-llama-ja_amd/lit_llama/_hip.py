@@ -88,9 +88,9 @@ SIGNATURES = {
     "llj_g_relu2": [_P, ctypes.c_size_t, _I, _P],
     "llj_gla_scan": [_P, _I, _I, _I, _I, _I, _I, _P, _I, _P, _I, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _F, _F, _F, _I,
                      _P],
-    "llj_rows_linear": [_I, _P, _I, _P, _P, _I, _I, _I, _I, _P],
+    "llj_rows_linear": [_I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _F, _F, _P],
     "llj_post_linear": [_I, _P, _P, _F, _P, _P, _I, _P, _P, _I, _I, _P],
-    "llj_gemm_bf16": [_I, _P, _I, _P, _P, _I, _I, _I, _I, _P, ctypes.c_size_t, _P],
+    "llj_gemm_bf16": [_I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _F, _F, _P, ctypes.c_size_t, _P],
     "llj_gla_chunk_rows": [_I, _I],
     "llj_gla_chunks": [_P, _I, _I, _I, _I, _I, _I, _P, _I, _P, _I, _P, _P, _I, _P, _P, _P, _I, _P, _I, _P, _P, _I, _I, _I,
                        _F, _F, _F, _I, _P],
@@ -106,6 +106,20 @@ SIGNATURES = {
     "llj_prev_commit": [_P, _P, _P, _P, _I, _P],
     "llj_latent_rows": [_P, _I, _I, _I, _P, _I, _P, _I, _P, _P, _I, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I,
                         _I, _I, _F, _I, _P],
+    "llj_g_bias_act": [_I, _P, _I, _P, _P, _I, _I, _I, _F, _F, _I, _P],
+    "llj_streams_embed": [_P, _P, _I, _F, _P, _P, _I, _I, _P, _P, _F, _P, _I, _I, _I, _I, _P],
+    "llj_streams_step": [_P, _I, _P, _P, _P, _I, _I, _P, _P, _F, _P, _I, _P, _I, _I, _I, _P],
+    "llj_streams_linear_ok": [_I, _I],
+    "llj_streams_linear": [_I, _P, _P, _P, _P, _P, _I, _I, _P, _P, _F, _I, _P, _P, _P, _I, _I, _F, _F, _P],
+    "llj_gqa_prep": [_P, _I, _I, _I, _I, _P, _I, _I, _F, _P, _P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I,
+                     _P],
+    "llj_gqa_rows": [_P, _I, _I, _I, _P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P],
+    "llj_gqa_flash_rows": [_I, _I, _I],
+    "llj_gqa_flash": [_P, _I, _I, _I, _P, _I, _I, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _F, _I, _P],
+    "llj_gqa_decode_ok": [_I, _I],
+    "llj_gqa_part_width": [_I],
+    "llj_gqa_decode": [_P, _I, _I, _I, _I, _I, _P, _I, _I, _F, _P, _P, _P, _I, _I, _P, _P, _I, _P, _I, _P, _I, _I,
+                       _I, _I, _I, _I, _F, _I, _P],
     "llj_g_i8_linear": [_P, _I, _I, _I, _P, _P, _F, _P, _I, _P, _I, _P, _I, _I, _P],
 }
 

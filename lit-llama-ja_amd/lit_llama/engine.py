@@ -17,7 +17,7 @@ rows share every fused launch; larger batches take the ops in row slices.
 The model-specific half of a session is its program (model.session_program(session)): what a prompt
 call and a decode step launch, and what they keep. LLaMAProgram drives the K / V cache models (one
 position shared by the rows); HybridProgram drives models with per-sequence state (state.SequenceState:
-recurrent states and latent rings behind a slot per sequence), whose prompts may differ in length and
+recurrent states, latent rings and K / V rows behind a slot per sequence), whose prompts may differ in length and
 whose sequences may end one by one (`finish`). `feed` runs a step on given tokens instead of the chosen
 ones.
 """
@@ -151,6 +151,11 @@ class HybridProgram:
         rows = Rows(s.B, s.B, s.cur, s.pos, self.slot)
         s.model.run(rows, s.work, self.state, s.logits, None, st)
 
+    def room(self, n: int) -> None:
+        """State for n more tokens per row."""
+        if self.state.ensure(max(self.seen) + n):
+            self.sess.graph = None
+
     def finish(self, live: list) -> None:
         kept = set(live)
         self.state.release([x for b, x in enumerate(self.slots) if b not in kept])
@@ -159,6 +164,7 @@ class HybridProgram:
     def extend(self, live: list, tokens: list, want) -> torch.Tensor:
         """These live rows take in their next tokens (one prompt-style call); the wanted places' logits."""
         s = self.sess
+        self.room(max(map(len, tokens)))
         out = s.model.extend(self.state, [self.slots[b] for b in live], [self.seen[b] for b in live], tokens, want)
         for b, t in zip(live, tokens):
             self.seen[b] += len(t)
@@ -251,6 +257,8 @@ class DecodeSession:
         assert self.total is None or self.t_prompt + self.steps_done + n <= self.total, "beyond the output buffer"
         limit = self.S if self.ragged and self.S is not None else self.model.config.block_size
         assert self.t_prompt + self.steps_done + n - 1 <= limit, "beyond block_size"
+        if self.ragged:
+            self.program.room(n)
         if self.use_graph:
             self.capture()
             for _ in range(n):

@@ -1,5 +1,5 @@
-"""Layer mechanisms shared by hybrid models: packed Linear groups, gated linear attention, latent attention
-and the squared-relu feed-forward. Each mixer reads one activation row per token and leaves its gated
+"""Layer mechanisms shared by hybrid models: packed Linear groups, gated linear attention, latent attention,
+grouped-query attention, and the squared-relu and clamped gated feed-forwards. Each mixer reads one activation row per token and leaves its gated
 output for its output projection; sizes and constants are parameters, the compute is the library's.
 
 Activation type: bfloat16 or float32; the residual, norms, gates of the recurrence, recurrent state and
@@ -13,6 +13,7 @@ from typing import Optional
 import torch
 
 from . import _hip
+from .state import ALL_POSITIONS
 from .utils import find_multiple
 
 GEMM_MIN_ROWS = 64  # bf16: from this many rows on the tiled prefill GEMM, below it slices of STREAM_ROWS
@@ -20,6 +21,9 @@ STREAM_ROWS = 16
 GLA_CHUNK_RANK = 240  # largest decay rank the chunked recurrence stages
 GLA_CHUNK_MIN = 16  # prompts with a sequence longer than this take the chunked recurrence
 ATTEND_WGS = 128  # latent decode attention: workgroups the visible keys of a batch are split for (one row: twice)
+GQA_WGS = 512  # grouped-query decode attention: workgroups the keys of a batch are split for
+GQA_RANGE = 128  # its shortest key range
+GQA_LONG = 1024  # prompts with a sequence this long take 128 queries per workgroup
 PART_ALIGN = 8  # output columns of the parts of a packed group start at multiples of this
 
 
@@ -35,9 +39,24 @@ def lane_pad(n: int, dtype) -> int:
 class PackedLinear:
     """Linear layers over the same input as one weight: rows of `parts` stacked (each part's first row
     at a multiple of PART_ALIGN), zero rows and columns up to the kernels' tiles. `offset[i]` is part i's
-    first output column."""
+    first output column. `biases`: one per part (None: none). `unit` = (limit, alpha): two parts of equal size, gate
+    and up, interleaved row by row, and the output is their clamped gated unit -- one column per pair, the
+    first lane_pad(part rows) columns."""
 
-    def __init__(self, parts: list, dtype, device):
+    def __init__(self, parts: list, dtype, device, biases: Optional[list] = None, unit: Optional[tuple] = None):
+        if unit is not None:
+            biases = biases or [None, None]
+            n, pad = parts[0].shape[0], lane_pad(parts[0].shape[0], dtype)
+            if len(parts) != 2 or parts[1].shape != parts[0].shape:
+                raise ValueError("a gated unit takes two parts of one shape")
+            both = torch.zeros(pad, 2, parts[0].shape[1], dtype=parts[0].dtype, device=parts[0].device)
+            bb = torch.zeros(pad, 2, dtype=torch.float32)
+            for j, (p, b) in enumerate(zip(parts, biases)):
+                both[:n, j] = p
+                if b is not None:
+                    bb[:n, j] = b.float().cpu()
+            parts, biases = [both.view(2 * pad, -1)], [bb.view(-1)]
+        self.unit = unit
         self.K = parts[0].shape[1]
         self.Kp = lane_pad(self.K, dtype)
         self.offset, n = [], 0
@@ -52,28 +71,45 @@ class PackedLinear:
         self.w = torch.zeros(self.Np, self.Kp, dtype=dtype, device=device)
         for o, p in zip(self.offset, parts):
             self.w[o:o + p.shape[0], :self.K] = p.to(device=device, dtype=dtype)
+        self.bias = None
+        if biases is not None and any(b is not None for b in biases):
+            v = torch.zeros(self.Np, dtype=torch.float32)
+            for o, p, b in zip(self.offset, parts, biases):
+                if b is not None:
+                    v[o:o + p.shape[0]] = b.float().cpu()
+            self.bias = v.to(device)
+        self.out_columns = self.Np // 2 if unit is not None else self.Np
 
     def nbytes(self) -> int:
         return self.w.numel() * self.w.element_size()
 
     def apply(self, a: torch.Tensor, M: int, out: torch.Tensor, st, relu2: bool = False) -> None:
-        """out[m, :Np] = a[m] . W^T for M rows (padding columns come out zero), optionally max(., 0)^2."""
-        if a.shape[1] < self.Kp or out.shape[1] < self.Np or a.shape[0] < M or out.shape[0] < M:
+        """out[m, :out_columns] = a[m] . W^T + bias for M rows (padding columns come out zero), through the gated unit,
+        or (layers without a bias) max(., 0)^2."""
+        if a.shape[1] < self.Kp or out.shape[1] < self.out_columns or a.shape[0] < M or out.shape[0] < M:
             raise ValueError(f"Linear ({self.Np}, {self.Kp}) on a {tuple(a.shape)} into {tuple(out.shape)}, {M} rows")
+        limit, alpha = self.unit or (0.0, 0.0)
+        act, bias = (2 if self.unit else int(relu2)), _hip.ptr(self.bias)
         if self.dtype == torch.float32:
+            y = torch.empty(M, self.Np, dtype=torch.float32, device=out.device) if self.unit else out
             _hip.call("llj_g_linear", 1, a.data_ptr(), a.stride(0), M, self.Kp, self.w.data_ptr(), None, None, 16, self.Kp,
-                      self.Np, out.data_ptr(), out.stride(0), None, 0, 1, st)
+                      self.Np, y.data_ptr(), y.stride(0), None, 0, 1, st)
+            if self.unit:
+                _hip.call("llj_g_bias_act", 2, y.data_ptr(), y.stride(0), bias, out.data_ptr(), out.stride(0), M, self.Np,
+                          limit, alpha, 1, st)
+            elif self.bias is not None:
+                _hip.call("llj_g_bias_act", 0, y.data_ptr(), y.stride(0), bias, None, 0, M, self.Np, 0.0, 0.0, 1, st)
             if relu2:
                 _hip.call("llj_g_relu2", out.data_ptr(), M * out.stride(0), 1, st)
         elif M < GEMM_MIN_ROWS:  # weight-streaming rows
             for r in range(0, M, STREAM_ROWS):
-                _hip.call("llj_rows_linear", int(relu2), a[r].data_ptr(), a.stride(0), self.w.data_ptr(), out[r].data_ptr(),
-                          out.stride(0), min(STREAM_ROWS, M - r), self.Np, self.Kp, st)
+                _hip.call("llj_rows_linear", act, a[r].data_ptr(), a.stride(0), self.w.data_ptr(), bias, out[r].data_ptr(),
+                          out.stride(0), min(STREAM_ROWS, M - r), self.Np, self.Kp, limit, alpha, st)
         else:
-            nb = 0 if relu2 else _hip.lib().llj_gemm_bf16_ws_bytes(M, self.Np, self.Kp)
+            nb = 0 if act else _hip.lib().llj_gemm_bf16_ws_bytes(M, self.Np, self.Kp)
             ws = torch.empty(nb // 4, dtype=torch.float32, device=out.device) if nb else None
-            _hip.call("llj_gemm_bf16", int(relu2), a.data_ptr(), a.stride(0), self.w.data_ptr(), out.data_ptr(),
-                      out.stride(0), M, self.Np, self.Kp, _hip.ptr(ws), nb, st)
+            _hip.call("llj_gemm_bf16", act, a.data_ptr(), a.stride(0), self.w.data_ptr(), bias, out.data_ptr(),
+                      out.stride(0), M, self.Np, self.Kp, limit, alpha, _hip.ptr(ws), nb, st)
 
     def takes_post(self, M: int, width: int) -> bool:
         """Whether apply_post serves these rows."""
@@ -86,10 +122,26 @@ class PackedLinear:
                   self.w.data_ptr(), out.data_ptr(), self.Np, self.Kp, st)
 
 
-def rotation_turns(dims: int, base: float, device) -> torch.Tensor:
-    """Frequencies base^(-2i / dims) of the interleaved rotation in turns per position, double precision."""
+    def takes_streams(self, M: int, width: int, streams: int) -> bool:
+        """Whether apply_streams serves these rows."""
+        return (self.dtype == torch.bfloat16 and M == 1 and width == self.K and
+                bool(_hip.lib().llj_streams_linear_ok(streams, width)))
+
+    def apply_streams(self, y: torch.Tensor, done, x: torch.Tensor, x_out: torch.Tensor, sub, eps: float, out: torch.Tensor,
+                      st) -> None:
+        """One row: the streams after sublayer `done` with its output y (x to x_out), read through sublayer `sub`'s
+        weights and norm, then this product, in one launch."""
+        limit, alpha = self.unit or (0.0, 0.0)
+        _hip.call("llj_streams_linear", 2 if self.unit else 0, y.data_ptr(), done.out.data_ptr(), done.mix.data_ptr(),
+                  x.data_ptr(), x_out.data_ptr(), x.shape[-1], x.shape[-2], sub.inp.data_ptr(), sub.norm.data_ptr(), eps,
+                  self.K, self.w.data_ptr(), _hip.ptr(self.bias), out.data_ptr(), self.Np, self.Kp, limit, alpha, st)
+
+
+def rotation_turns(dims: int, base: float, device, factor: float = 1.0) -> torch.Tensor:
+    """Frequencies base^(-2i / dims) / factor of a rotation's pairs in turns per position, double precision."""
     i = torch.arange(0, dims, 2, dtype=torch.float64)
-    return (torch.pow(torch.tensor(float(base), dtype=torch.float64), -i / dims) / (2.0 * torch.pi)).to(device)
+    f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -i / dims) / factor
+    return (f / (2.0 * torch.pi)).to(device)
 
 
 # ------------------------------------------------------------------------------------ gated linear attention
@@ -309,6 +361,117 @@ class LatentAttention:
                       rows.slot.data_ptr(), rows.M, _dt(self.dtype), st)
 
 
+# ------------------------------------------------------------------------------------ grouped-query attention
+@dataclass(frozen=True)
+class GroupedSpec:
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot_dims: int
+    rot_base: float
+    rot_factor: float = 1.0  # divides the rotation's frequencies
+    v_mix: bool = False  # values mixed with those of the first such layer
+    qk_norm: bool = True  # rotated queries and keys divided by their root mean square
+    sink: bool = True  # a key of score 0 without a value
+
+
+class GroupedAttention:
+    """Causal grouped-query attention with biased projections, rotate-half positions and one sigmoid gate per
+    head (csrc/gqa.hip). Keeps a K / V row of every token (state.ALL_POSITIONS)."""
+
+    def __init__(self, spec: GroupedSpec, width: int, eps: float):
+        self.spec, self.width, self.eps = spec, width, eps
+        self.first: Optional[GroupedAttention] = None  # v_mix: the layer whose values are mixed in (itself: it leaves them)
+
+    def shapes(self) -> dict:
+        s, C = self.spec, self.width
+        out = {"q": (s.heads * s.dim, C), "k": (s.kv_heads * s.dim, C), "v": (s.kv_heads * s.vdim, C), "g": (s.heads, C),
+               "o": (C, s.heads * s.vdim)}
+        out.update({n + ".b": (out[n][0],) for n in "qkvo"})
+        if s.v_mix:
+            out["vmix"] = ()
+        return out
+
+    def load(self, t: dict, dtype, device) -> None:
+        s = self.spec
+        if not s.v_mix:
+            t.pop("vmix", None)
+        _check_shapes(t, self.shapes())
+        self.inp = PackedLinear([t["q"], t["k"], t["v"], t["g"]], dtype, device, [t["q.b"], t["k.b"], t["v.b"], None])
+        self.out = PackedLinear([t["o"]], dtype, device, [t["o.b"]])
+        self.lam = t["vmix"].to(device=device, dtype=torch.float32).reshape(1) if s.v_mix and self.first is not self else None
+        self.turns = rotation_turns(s.rot_dims, s.rot_base, device, s.rot_factor)
+        self.dtype = dtype
+
+    def linears(self) -> list:
+        return [self.inp, self.out]
+
+    def state_shape(self):
+        return None
+
+    def ring_window(self):
+        return ALL_POSITIONS
+
+    def cache_width(self, dtype) -> int:
+        return find_multiple(self.spec.kv_heads * (self.spec.dim + self.spec.vdim), 8)
+
+    def out_width(self) -> int:
+        return self.spec.heads * self.spec.vdim
+
+    def first_width(self) -> int:
+        """Columns of the values the first mixing layer leaves for the others."""
+        return self.spec.kv_heads * self.spec.vdim if self.spec.v_mix else 0
+
+    def _decode_ok(self) -> bool:
+        s = self.spec
+        return self.dtype == torch.bfloat16 and bool(_hip.lib().llj_gqa_decode_ok(s.dim, s.vdim))
+
+    def _splits(self, M: int, W: int) -> int:
+        """Key ranges of a decode step over a cache of W rows (None: the most there can be)."""
+        s = self.spec
+        most = max(1, min(64, GQA_WGS // (M * s.kv_heads * ((s.heads // s.kv_heads + 15) // 16))))
+        return most if W is None else max(1, min(most, (W + GQA_RANGE - 1) // GQA_RANGE))
+
+    def _part(self, w, M: int, n: int):
+        s = self.spec
+        return w.buffer("part", M * s.heads * n * _hip.lib().llj_gqa_part_width(s.vdim), torch.float32)
+
+    def reserve(self, w, M: int) -> None:
+        if self._decode_ok():
+            self._part(w, M, self._splits(M, None))
+
+    def mix(self, i: int, rows, w, state, y: torch.Tensor, st) -> None:
+        """y = gated output of layer i from the packed projections w.proj; the rows' keys and values into the state."""
+        s, p, o, M = self.spec, w.proj, self.inp.offset, rows.M
+        cache, W, ldc = state.ring[i], state.ring_rows[i], self.cache_width(self.dtype)
+        first = w.first if s.v_mix else None
+        new = (self.turns.data_ptr(), s.rot_dims, int(s.qk_norm), self.eps)
+        mixed = (_hip.ptr(first), _hip.ptr(self.lam), 0 if first is None else first.stride(0))
+        sizes = (M, s.heads, s.kv_heads, s.dim, s.vdim)
+        if rows.decode and self._decode_ok():
+            n = self._splits(M, W)
+            _hip.call("llj_gqa_decode", p.data_ptr(), p.stride(0), o[0], o[1], o[2], o[3], *new, rows.pos.data_ptr(),
+                      rows.slot.data_ptr(), cache.data_ptr(), W, ldc, *mixed, self._part(w, M, n).data_ptr(), n,
+                      y.data_ptr(), y.stride(0), *sizes, s.scale, int(s.sink), st)
+            return
+        _hip.call("llj_gqa_prep", p.data_ptr(), p.stride(0), o[0], o[1], o[2], *new, rows.pos.data_ptr(),
+                  _hip.ptr(rows.row_seq), rows.slot.data_ptr(), cache.data_ptr(), W, ldc, *mixed, *sizes, _dt(self.dtype), st)
+        C = 0
+        if not rows.decode and self.dtype == torch.bfloat16:
+            C = _hip.lib().llj_gqa_flash_rows(s.dim, s.vdim, int(max(rows.lengths) >= GQA_LONG))
+        if C:
+            n, work = rows.pairs(C)
+            _hip.call("llj_gqa_flash", p.data_ptr(), p.stride(0), o[0], o[3], work.data_ptr(), n, C, rows.pos.data_ptr(),
+                      rows.slot.data_ptr(), cache.data_ptr(), W, ldc, y.data_ptr(), y.stride(0), *sizes, s.scale,
+                      int(s.sink), st)
+            return
+        _hip.call("llj_gqa_rows", p.data_ptr(), p.stride(0), o[0], o[3], rows.pos.data_ptr(), _hip.ptr(rows.row_seq),
+                  rows.slot.data_ptr(), cache.data_ptr(), W, ldc, y.data_ptr(), y.stride(0), *sizes, s.scale, int(s.sink),
+                  _dt(self.dtype), st)
+
+
 # ------------------------------------------------------------------------------------ feed-forward
 class ReluSquaredMLP:
     """W_down max(W_up h, 0)^2"""
@@ -326,6 +489,37 @@ class ReluSquaredMLP:
 
     def linears(self) -> list:
         return [self.up, self.down]
+
+
+class ClampedGLU:
+    """W_down of the clamped gated unit (PackedLinear's `unit`) of W_gate h and W_up h, all biased."""
+
+    def __init__(self, ff: int, width: int, limit: float, alpha: float):
+        self.ff, self.width, self.unit = ff, width, (limit, alpha)
+
+    def shapes(self) -> dict:
+        F, C = self.ff, self.width
+        return {"gate": (F, C), "gate.b": (F,), "up": (F, C), "up.b": (F,), "down": (C, F), "down.b": (C,)}
+
+    def load(self, t: dict, dtype, device) -> None:
+        _check_shapes(t, self.shapes())
+        self.up = PackedLinear([t["gate"], t["up"]], dtype, device, [t["gate.b"], t["up.b"]], unit=self.unit)
+        self.down = PackedLinear([t["down"]], dtype, device, [t["down.b"]])
+
+    def linears(self) -> list:
+        return [self.up, self.down]
+
+
+# ------------------------------------------------------------------------------------ residual streams
+@dataclass
+class StreamSublayer:
+    """How a sublayer reads and leaves the residual streams (csrc/streams.hip): u = sum_s inp[s] x_s through a layer
+    norm with weight `norm`, then x_t = sum_s mix[s, t] x_s + out[t] y."""
+
+    inp: torch.Tensor
+    out: torch.Tensor
+    mix: torch.Tensor
+    norm: torch.Tensor
 
 
 def _check_shapes(t: dict, want: dict) -> None:

@@ -19,40 +19,12 @@ from typing import Optional, Tuple
 import torch
 
 from . import _hip
+from .hybrid import MAX_POSITIONS, HybridModel, Scratch, TensorReader, take_values
 from .mixers import (GatedLinearAttention, GLASpec, LatentAttention, LatentSpec, PackedLinear, ReluSquaredMLP, _dt,
                      lane_pad)
 from .registry import register
 from .state import Rows, SequenceState
 from .utils import find_multiple
-
-MAX_POSITIONS = 1 << 30  # positions are int32; the layers themselves have no length limit
-
-
-def _take(d: dict, where: str, **kinds) -> list:
-    """Values of a config object with exactly these keys; a kind with a default (kind, default) is optional."""
-    if not isinstance(d, dict):
-        raise ValueError(f"config: {where} is not an object")
-    extra = set(d) - set(kinds)
-    if extra:
-        raise ValueError(f"config: {where} has unknown keys {sorted(extra)}")
-    out = []
-    for key, kind in kinds.items():
-        default = ()
-        if isinstance(kind, tuple):
-            kind, default = kind[0], kind[1:]
-        if key not in d:
-            if not default:
-                raise ValueError(f"config: {where} has no '{key}'")
-            out.append(default[0])
-            continue
-        v = d[key]
-        if v is None and default == (None,):
-            out.append(None)
-            continue
-        if kind is int and (isinstance(v, bool) or int(v) != v):
-            raise ValueError(f"config: {where}.{key} is not an integer")
-        out.append(kind(v) if kind in (int, float) else v)
-    return out
 
 
 @dataclass(frozen=True)
@@ -83,23 +55,23 @@ class MugivikConfig:
 
     @classmethod
     def from_dict(cls, d: dict) -> "MugivikConfig":
-        _, emb, layers, norm, vocab, width = _take(d, "config.json", architecture=str, embedding=dict, layers=list,
-                                                   norm=dict, vocab=int, width=int)
-        (big,) = _take(emb, "embedding", bigram=dict)
-        buckets, mc, mp = _take(big, "embedding.bigram", buckets=int, mul_cur=int, mul_prev=int)
-        (eps,) = _take(norm, "norm", eps=float)
+        _, emb, layers, norm, vocab, width = take_values(d, "config.json", architecture=str, embedding=dict, layers=list,
+                                                         norm=dict, vocab=int, width=int)
+        (big,) = take_values(emb, "embedding", bigram=dict)
+        buckets, mc, mp = take_values(big, "embedding.bigram", buckets=int, mul_cur=int, mul_prev=int)
+        (eps,) = take_values(norm, "norm", eps=float)
         out = []
         for i, layer in enumerate(layers):
             where = f"layers[{i}]"
-            mix, mlp, kind = _take(layer, where, mixer=dict, mlp=(dict, None), type=str)
+            mix, mlp, kind = take_values(layer, where, mixer=dict, mlp=(dict, None), type=str)
             if kind == "gla":
-                spec = GLASpec(*_take(mix, where + ".mixer", heads=int, dim=int, vdim=int, tau=float))
+                spec = GLASpec(*take_values(mix, where + ".mixer", heads=int, dim=int, vdim=int, tau=float))
             elif kind == "latent_attention":
-                heads, dim, rd, vdim, rank, mask, scale, rot, src = _take(
+                heads, dim, rd, vdim, rank, mask, scale, rot, src = take_values(
                     mix, where + ".mixer", heads=int, dim=int, rot_dim=int, vdim=int, kv_rank=int, mask=dict, scale=float,
                     rot=dict, kv_from=(int, None))
-                (window,) = _take(mask, where + ".mixer.mask", size=int)
-                base, dims = _take(rot, where + ".mixer.rot", base=float, dims=int)
+                (window,) = take_values(mask, where + ".mixer.mask", size=int)
+                base, dims = take_values(rot, where + ".mixer.rot", base=float, dims=int)
                 if dims != rd:
                     raise ValueError(f"config: {where} rotates {dims} of rot_dim {rd} dimensions")
                 if src is not None and not 0 <= src < i:
@@ -111,7 +83,7 @@ class MugivikConfig:
                 raise ValueError(f"config: {where} has unknown type {kind!r}")
             ff = None
             if mlp is not None:
-                ff, mk = _take(mlp, where + ".mlp", ff=int, kind=str)
+                ff, mk = take_values(mlp, where + ".mlp", ff=int, kind=str)
                 if mk != "dense":
                     raise ValueError(f"config: {where}.mlp has unknown kind {mk!r}")
             out.append(MugivikLayer(spec, ff))
@@ -120,11 +92,10 @@ class MugivikConfig:
         return cls(vocab, width, eps, buckets, mp, mc, tuple(out))
 
 
-class _Work:
-    """Scratch of a forward call over M rows (a decode session keeps one for all its steps)."""
-
+class _Work(Scratch):
     def __init__(self, m: "Mugivik", M: int):
         dev, dt, C = m.device, m.dtype, m.Cp
+        super().__init__(M, dev)
         self.x = torch.empty(M, C, dtype=torch.float32, device=dev)
         # the sublayers' input: the residual itself in float32, its bf16 copy otherwise
         self.xb = self.x if dt == torch.float32 else torch.empty(M, C, dtype=dt, device=dev)
@@ -137,21 +108,11 @@ class _Work:
         # mixer outputs by width: padding columns stay zero
         self.y = {n: torch.zeros(M, lane_pad(n, dt), dtype=dt, device=dev) for n in {mx.out_width() for mx in m.mixers}}
         self.cur: dict = {}  # this call's latents by layer (prompt rows)
-        self.all_rows = torch.arange(M, dtype=torch.int32, device=dev)
-        self.hb = None  # the head's input rows
         self.x2 = torch.empty_like(self.x) if M == 1 else None  # the residual's other place (fused post-norm products)
-        self._buffers: dict = {}
-
-    def buffer(self, name: str, numel: int, dtype) -> torch.Tensor:
-        """Scratch shared by the layers, at least numel long."""
-        t = self._buffers.get(name)
-        if t is None or t.numel() < numel:
-            t = self._buffers[name] = torch.empty(numel, dtype=dtype, device=self.x.device)
-        return t
 
 
 @register("Mugivik")
-class Mugivik(torch.nn.Module):
+class Mugivik(HybridModel):
     HIP_SOURCES = ("postnorm", "post_gemv", "gemm_bf16", "gla", "latent", "latent_prefill", "latent_decode", "generic",
                    "ops", "options")
 
@@ -195,26 +156,16 @@ class Mugivik(torch.nn.Module):
             raise TypeError(f"Mugivik computes in bfloat16 or float32, not {dtype}")
         m = cls(config)
         m.dtype, m.device = dtype, torch.device(device)
-        left = dict(tensors)
-
-        def take(name, shape):
-            if name not in left:
-                raise ValueError(f"tensor {name} is missing")
-            t = left.pop(name)
-            if tuple(t.shape) != tuple(shape):
-                raise ValueError(f"tensor {name} has shape {tuple(t.shape)}, expected {tuple(shape)}")
-            return t
+        src = TensorReader(tensors)
+        take, group = src.take, src.group
 
         def vec(name):
             return take(name, (config.n_embd,)).to(device=m.device, dtype=dtype).contiguous()
 
-        def group(prefix):
-            return {k[len(prefix):]: left.pop(k) for k in [n for n in left if n.startswith(prefix)]}
-
         C = config.n_embd
         m.Cp = lane_pad(C, dtype)
         # one copy of the table for the lookup and the tied head
-        m.embed = PackedLinear([take("embed", (config.vocab_size, C))], dtype, m.device)
+        m.embed = m.head = PackedLinear([take("embed", (config.vocab_size, C))], dtype, m.device)
         m.bigram = take("bigram", (config.buckets + 1, C)).to(device=m.device, dtype=dtype).contiguous()
         m.embed_norm, m.final_norm = vec("embed.norm"), vec("final.norm")
         m.norm1, m.norm2 = [], []
@@ -224,8 +175,7 @@ class Mugivik(torch.nn.Module):
             m.norm2.append(None if ml is None else vec(f"l{i}.norm2"))
             if ml is not None:
                 ml.load(group(f"l{i}.mlp."), dtype, m.device)
-        if left:
-            raise ValueError(f"unexpected tensors {sorted(left)}")
+        src.done()
         return m
 
     @classmethod
@@ -243,21 +193,10 @@ class Mugivik(torch.nn.Module):
                 t[name] = (r * shape[1] ** -0.5).to(dtype)
         return cls.from_tensors(config, t, dtype, device)
 
-    def session_program(self, sess):
-        from .engine import HybridProgram
-
-        return HybridProgram(sess)
-
-    def act_dtype(self) -> torch.dtype:
-        return self.dtype
-
-    def new_state(self, slots: int, max_length: Optional[int] = None) -> SequenceState:
-        return SequenceState(self, slots, max_length)
-
     def new_work(self, M: int, head_rows: int = 0) -> _Work:
         w = _Work(self, M)
         if head_rows:  # before a capture: nothing is allocated by the step itself
-            w.hb = torch.empty(head_rows, self.Cp, dtype=self.dtype, device=self.device)
+            w.head_rows(head_rows, self.Cp, self.dtype)
             for mx in self.mixers:
                 mx.reserve(w, M)
         return w
@@ -318,9 +257,7 @@ class Mugivik(torch.nn.Module):
                     pending = norm
         n = M if pick is None else pick.numel()
         if n:
-            if w.hb is None or w.hb.shape[0] < n:
-                w.hb = torch.empty(n, self.Cp, dtype=self.dtype, device=self.device)
-            hb, rows_idx = w.hb, w.all_rows if pick is None else pick
+            hb, rows_idx = w.head_rows(n, self.Cp, self.dtype), w.all_rows if pick is None else pick
             _hip.call("llj_post_norm", w.t.data_ptr(), self.Cp, pending.data_ptr(), eps, x.data_ptr(), self.Cp, hb.data_ptr(),
                       self.Cp, self.final_norm.data_ptr(), rows_idx.data_ptr(), n, C, _dt(self.dtype), st)
             self.embed.apply(hb, n, logits, st)
@@ -330,57 +267,3 @@ class Mugivik(torch.nn.Module):
                     mx.commit(i, rows, w, state, st)
             _hip.call("llj_prev_commit", rows.tok.data_ptr(), rows.row0.data_ptr(), rows.slot.data_ptr(),
                       state.prev.data_ptr(), rows.B, st)
-
-    def check_tokens(self, tokens) -> None:
-        if len(tokens) and not 0 <= min(tokens) <= max(tokens) < self.config.vocab_size:
-            raise ValueError(f"token ids must be in [0, {self.config.vocab_size})")
-
-    @torch.no_grad()
-    def extend(self, state: SequenceState, slots: list, starts: list, tokens: list, want: Optional[list] = None,
-               taps: Optional[list] = None) -> torch.Tensor:
-        """Run each sequence's next tokens (lists of ids) from its state. Returns the logits (n, vocab) at
-        the wanted places, want[b] a list of indices into tokens[b] (None: all), in that order."""
-        for t in tokens:
-            self.check_tokens(t)
-        rows = Rows.packed(tokens, starts, slots, self.device)
-        if want is None:
-            pick, n = None, rows.M
-        else:
-            base, idx = 0, []
-            for t, ks in zip(tokens, want):
-                if ks and not 0 <= min(ks) <= max(ks) < len(t):
-                    raise ValueError("wanted places must be among the tokens given")
-                idx += [base + k for k in ks]
-                base += len(t)
-            pick, n = torch.tensor(idx, dtype=torch.int32).to(self.device), len(idx)
-        logits = torch.empty(n, self.embed.Np, dtype=self.dtype, device=self.device)
-        self.run(rows, _Work(self, rows.M), state, logits, pick, _hip.stream(), taps)
-        return logits[:, :self.config.vocab_size]
-
-    @torch.no_grad()
-    def forward(self, idx: torch.Tensor, max_seq_length: Optional[int] = None,
-                input_pos: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """Logits (B, T, vocab) of B equal-length sequences, as LLaMA.forward: without input_pos from their
-        first token on a state of their own; with it (contiguous positions) going on from the model's
-        kept state, which the call with position 0 begins (reset_cache() ends it)."""
-        B, T = idx.shape
-        toks = idx.tolist()
-        if input_pos is None:
-            state = self.new_state(B, T)
-            return self.extend(state, state.alloc(B), [0] * B, toks).view(B, T, -1)
-        p = input_pos.tolist()
-        if p != list(range(p[0], p[0] + T)):
-            raise ValueError("input_pos must be T contiguous positions")
-        if getattr(self, "_kept", None) is None:
-            if p[0] != 0:
-                raise ValueError("the first call with input_pos must begin at position 0")
-            self._kept = (state := self.new_state(B, max_seq_length), state.alloc(B), [0] * B)
-        state, slots, seen = self._kept
-        if len(slots) != B or seen[0] != p[0]:
-            raise ValueError(f"expected {len(slots)} sequences at position {seen[0]}; call reset_cache() first")
-        out = self.extend(state, slots, seen, toks).view(B, T, -1)
-        self._kept = (state, slots, [p[0] + T] * B)
-        return out
-
-    def reset_cache(self) -> None:
-        self._kept = None

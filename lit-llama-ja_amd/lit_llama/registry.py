@@ -34,7 +34,7 @@ def architectures() -> list:
 
 
 def _load_all() -> None:
-    from . import model, mugivik  # noqa: F401  (they register themselves)
+    from . import bobasun, model, mugivik  # noqa: F401  (they register themselves)
 
 
 def model_class(name: str):

@@ -4,6 +4,8 @@
   * every recurrent layer's state (fp32, mixer.state_shape),
   * every latent-attention layer's ring of the last tokens' latents, one per layer that projects its own
     (layers that read another layer's latents have none), sized by the widest window among its readers,
+  * every full-attention layer's K / V rows, the same buffers with a row for every position: as many as the
+    longest sequence allowed, or without a limit as many as the longest has needed so far (`ensure`),
   * the previous token of each sequence (models whose embedding looks back one token).
 A sequence holds a slot from `alloc` to `release`; kernels address everything through the slot number, so
 the rows of a batch need not be neighbours in memory and a batch can shrink without moving state.
@@ -11,6 +13,9 @@ the rows of a batch need not be neighbours in memory and a batch can shrink with
 from __future__ import annotations
 
 import torch
+
+ALL_POSITIONS = -1  # mixer.ring_window() of layers that keep every token
+GROW_ROWS = 256  # unlimited layers grow by multiples of this many rows
 
 
 class SequenceState:
@@ -23,8 +28,11 @@ class SequenceState:
         self.ring_rows: dict = {}
         for i, mixer in enumerate(model.mixers):
             w = mixer.ring_window()
-            if w is not None:
+            if w == ALL_POSITIONS:
+                self.ring_rows[i] = 0 if max_length is None else max(1, max_length)
+            elif w is not None:
                 self.ring_rows[i] = w if max_length is None else max(1, min(w, max_length))
+        self._all = [i for i, mixer in enumerate(model.mixers) if mixer.ring_window() == ALL_POSITIONS]
         self._free: list = []
         self._grow(slots)
 
@@ -39,6 +47,21 @@ class SequenceState:
         self.prev = torch.full((slots,), -1, dtype=torch.int32, device=dev)
         self._free = list(range(slots))
         self.slots = slots
+
+    def ensure(self, length: int) -> bool:
+        """Room for sequences of `length` tokens in the layers that keep every token; True if they moved (a captured
+        step must be captured again)."""
+        if not self._all or length <= self.ring_rows[self._all[0]]:
+            return False
+        if self.max_length is not None:
+            raise ValueError(f"sequence of {length} tokens in a state for {self.max_length}")
+        rows = max(-(-length // GROW_ROWS) * GROW_ROWS, 2 * self.ring_rows[self._all[0]])
+        for i in self._all:
+            old = self.ring[i]
+            new = torch.zeros(old.shape[0], rows, old.shape[2], dtype=old.dtype, device=old.device)
+            new[:, :old.shape[1]] = old
+            self.ring[i], self.ring_rows[i] = new, rows
+        return True
 
     def reserve(self, n: int) -> None:
         """Room for n more sequences; only an idle state can grow."""
@@ -124,6 +147,32 @@ class Rows:
             return len(tab) // 3, d[:len(tab)], d[len(tab):]
 
         return self._table(("chunks", C), make)
+
+    def pairs(self, C: int):
+        """Work items of causal attention over blocks of at most C rows of one sequence: (number, table [(first row,
+        rows, sequence) twice]) -- a late block, which sees many keys, with an early one (rows 0: none)."""
+
+        def make():
+            tab, row = [], 0
+            for b, n in enumerate(self.lengths):
+                blocks = [[row + j, min(C, n - j), b] for j in range(0, n, C)]
+                row += n
+                while blocks:
+                    late = blocks.pop()
+                    tab.append(late + (blocks.pop(0) if blocks else [0, 0, 0]))
+            # the items with the most keys first
+            pos = [s - r0 for s, r0 in zip(self.starts, self._row0())]
+            tab.sort(key=lambda w: -(pos[w[2]] + w[0] + w[1]))
+            return len(tab), self._device([x for w in tab for x in w])
+
+        return self._table(("pairs", C), make)
+
+    def _row0(self) -> list:
+        out, row = [], 0
+        for n in self.lengths:
+            out.append(row)
+            row += n
+        return out
 
     def keys(self, window: int):
         """The keys the packed rows of a call may see through `window`: (number, gather or None, key0, kpos0,

@@ -94,7 +94,7 @@ def test_rows_linear(hip, M, N, K, act):
     A = torch.randn(M, K + 8, generator=g, device="cuda").to(torch.bfloat16)
     W = (torch.randn(N, K, generator=g, device="cuda") * K ** -0.5).to(torch.bfloat16)
     out = torch.full((M, N + 16), 3.0, dtype=torch.bfloat16, device="cuda")
-    call("llj_rows_linear", act, A, K + 8, W, out, N + 16, M, N, K)
+    call("llj_rows_linear", act, A, K + 8, W, None, out, N + 16, M, N, K, 0.0, 0.0)
     want = back(A)[:, :K] @ back(W).T
     want = np.maximum(want, 0) ** 2 if act else want
     close(back(out)[:, :N], want, 5e-3)
@@ -131,7 +131,7 @@ def test_gemm_bf16(hip, M, N, K, act):
     want = np.maximum(want, 0) ** 2 if act else want
     for ws in {None, nb or None}:
         buf = None if ws is None else torch.empty(nb // 4, device="cuda")
-        call("llj_gemm_bf16", act, A, K, W, out, N, M, N, K, buf, nb)
+        call("llj_gemm_bf16", act, A, K, W, None, out, N, M, N, K, 0.0, 0.0, buf, nb)
         close(back(out), want, 5e-3, ws)
 
 

@@ -121,7 +121,7 @@ def test_safetensors_reader(tmp_path):
 def test_registry():
     from lit_llama import registry
 
-    assert registry.architectures() == ["LLaMA", "Mugivik"]
+    assert registry.architectures() == ["Bobasun", "LLaMA", "Mugivik"]
     with pytest.raises(ValueError):
         registry.model_class("Other")
     c = registry.model_class("LLaMA").config_from_dict({"architecture": "LLaMA", "n_layer": 2, "n_head": 4, "n_embd": 64})
