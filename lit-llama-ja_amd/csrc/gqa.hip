@@ -417,47 +417,74 @@ __global__ __launch_bounds__(256) void gqa_attend_kernel(GqaParams p, float* __r
       vr[i] = *reinterpret_cast<const u32x4*>(vb + (size_t)(key < ps ? key : ps) * p.ldc + (c < V ? c : 0));
     }
   };
+  // ---- queries and the new key: 16 lanes per head; their loads first (a lane's items as in the preparation kernel: pairs,
+  // then unrotated dimensions), then the first step's keys and values, all in flight over the angles
+  const bf16_t* row = (const bf16_t*)p.in + (size_t)m * p.ld;
+  constexpr int NI = 2 * KT;  // items per lane, at most
+  const int hh = tid >> 4, l = tid & 15, items = n + D - p.RD;
+  const bool qlive = hh < nh;
+  bf16_t qa[NI], qc[NI], ka[NI], kc[NI];
+  auto place = [&](int j, int& k, bool& pair) {  // (items past the end read a valid place and are dropped)
+    const int it = l + 16 * j;
+    pair = it < n;
+    k = pair ? it : p.RD + it - n;
+    const bool in = it < items;
+    k = in ? k : 0;
+    return in;
+  };
+  {
+    const bf16_t* qs = row + p.oq + (h0 + (qlive ? hh : 0)) * D;
+    const bf16_t* ks = row + p.ok + gh * D;
+#pragma unroll
+    for (int j = 0; j < NI; ++j) {
+      int k;
+      bool pair;
+      place(j, k, pair);
+      qa[j] = qs[k];
+      qc[j] = qs[pair ? k + n : k];
+      ka[j] = ks[k];
+      kc[j] = ks[pair ? k + n : k];
+    }
+  }
   if (s0 + wave < s1) fetch(s0 + wave);
-  // ---- queries and the new key: 16 lanes per head, scalar items as in the preparation kernel
   for (int i = tid; i < n; i += 256) turn_cs(p.turns, i, ps, cs[i], cs[n + i]);
   for (int i = tid; i < 17 * QP / 8; i += 256) *reinterpret_cast<u32x4*>(Qs + 8 * i) = zero;
   __syncthreads();
-  const bf16_t* row = (const bf16_t*)p.in + (size_t)m * p.ld;
-  for (int q = 0; q < (owner ? 2 : 1); ++q) {
-    const int hh = tid >> 4, l = tid & 15;  // q = 1: group 0 takes the key
-    const bool live = q ? hh == 0 : hh < nh;
-    const bf16_t* src = row + (q ? p.ok + gh * D : p.oq + (h0 + (live ? hh : 0)) * D);
-    bf16_t* out = q ? Kn : Qs + hh * QP;
-    const int items = n + D - p.RD;
-    float ss = 0.f;
-    for (int pass = 0; pass < 2; ++pass) {
-      float r = 1.f;
-      if (pass) {
-        ss = row16_sum(ss);
-        if (p.qk_norm) r = 1.f / sqrtf(ss / (float)D + p.eps);
+  auto prepare = [&](const bf16_t (&a)[NI], const bf16_t (&c)[NI], bool live, bf16_t* out, bf16_t* out2) {
+    float u[NI], v[NI], ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < NI; ++j) {
+      int k;
+      bool pair;
+      const bool in = place(j, k, pair);
+      u[j] = bf2f(a[j]);
+      v[j] = 0.f;
+      if (pair) {
+        const float x = u[j], y = bf2f(c[j]), co = cs[k], si = cs[n + k];
+        u[j] = x * co - y * si;
+        v[j] = y * co + x * si;
       }
-      for (int it = l; live && it < items; it += 16) {
-        const bool pair = it < n;
-        const int k = pair ? it : p.RD + it - n;
-        float a = bf2f(src[k]), c = 0.f;
-        if (pair) {
-          const float v = bf2f(src[k + n]), u = a;
-          a = u * cs[k] - v * cs[n + k];
-          c = v * cs[k] + u * cs[n + k];
-        }
-        if (!pass) {
-          ss += a * a + c * c;
-        } else {
-          out[k] = f2bf(a * r);
-          if (pair) out[k + n] = f2bf(c * r);
-          if (q) {
-            kb[(size_t)ps * p.ldc + k] = f2bf(a * r);
-            if (pair) kb[(size_t)ps * p.ldc + k + n] = f2bf(c * r);
-          }
+      ss += in ? u[j] * u[j] + v[j] * v[j] : 0.f;
+    }
+    ss = row16_sum(ss);
+    const float r = p.qk_norm ? 1.f / sqrtf(ss / (float)D + p.eps) : 1.f;
+#pragma unroll
+    for (int j = 0; j < NI; ++j) {
+      int k;
+      bool pair;
+      if (place(j, k, pair) && live) {
+        const bf16_t x = f2bf(u[j] * r), y = f2bf(v[j] * r);
+        out[k] = x;
+        if (pair) out[k + n] = y;
+        if (out2) {
+          out2[k] = x;
+          if (pair) out2[k + n] = y;
         }
       }
     }
-  }
+  };
+  prepare(qa, qc, qlive, Qs + hh * QP, nullptr);
+  if (owner && wave == 0) prepare(ka, kc, hh == 0, Kn, kb + (size_t)ps * p.ldc);
   if (owner && tid < VW) {
     bf16_t o = 0;
     if (tid < V) {
@@ -645,7 +672,7 @@ static int gqa_check(const GqaParams& p) {
   return 0;
 }
 static int gqa_check_new(const GqaParams& p) {
-  LLJ_REQUIRE(p.turns && p.RD >= 0 && p.RD % 2 == 0 && p.RD <= p.D && p.ok >= 0 && p.ok + p.G * p.D <= p.ld && p.ov >= 0 &&
+  LLJ_REQUIRE((p.turns || !p.RD) && p.RD >= 0 && p.RD % 2 == 0 && p.RD <= p.D && p.ok >= 0 && p.ok + p.G * p.D <= p.ld && p.ov >= 0 &&
               p.ov + p.G * p.V <= p.ld && (!p.lam || p.first) && (!p.first || p.ldf >= p.G * p.V));
   return 0;
 }

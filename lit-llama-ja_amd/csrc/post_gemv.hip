@@ -253,11 +253,13 @@ static int post_gemv_go(const PostGemvParams& p, int act, hipStream_t s) {
 #ifndef LLJ_PG_HALF_M
 #define LLJ_PG_HALF_M 8  // largest row count that takes the half-K form where it applies (A/B; 0: never)
 #endif
+static int post_threads(int K) { return K > 4096 ? 512 : 256; }
+
 template <int NV, bool STREAMS = false>
 static int post_gemv_launch(const PostGemvParams& p, int act, hipStream_t s) {
   const bool half = p.M <= LLJ_PG_HALF_M && p.N / 16 < 256 && p.K % 256 == 0 && p.K >= 1024;
   if constexpr (NV > 0) {  // (the thread count is post_threads')
-    if (p.K > 4096)
+    if (post_threads(p.K) == 512)
       return half ? post_gemv_go<8, 4, NV, true, STREAMS>(p, act, s) : post_gemv_go<8, 4, NV, false, STREAMS>(p, act, s);
     return half ? post_gemv_go<4, 4, NV, true, STREAMS>(p, act, s) : post_gemv_go<4, 4, NV, false, STREAMS>(p, act, s);
   } else {
@@ -267,8 +269,6 @@ static int post_gemv_launch(const PostGemvParams& p, int act, hipStream_t s) {
     return p.K > 2048 ? post_gemv_go<8, 4, 0, false, false>(p, act, s) : post_gemv_go<4, 4, 0, false, false>(p, act, s);
   }
 }
-
-static int post_threads(int K) { return K > 4096 ? 512 : 256; }
 
 }  // namespace llj
 

@@ -31,88 +31,115 @@ struct StreamsParams {
   int S, C;
 };
 
-__device__ __forceinline__ float block_sum4(float v, float* red) {
+constexpr int kFewRows = 64;
+
+template <int NW>
+__device__ __forceinline__ float block_sum(float v, float* red) {
   v = wave_sum(v);
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
   __syncthreads();
-  const float s = red[0] + red[1] + red[2] + red[3];
+  float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < NW; ++i) s += red[i];
   __syncthreads();
   return s;
 }
 
-// One workgroup per row, 8 columns per thread and step, the widths up to 8 * 256 * NV held in registers.
-template <typename T, int S, int NV>
-__global__ __launch_bounds__(256) void streams_kernel(StreamsParams p) {
-  __shared__ float red[4];
+// VW (8 or 4) consecutive elements
+template <int VW, typename T>
+__device__ __forceinline__ void ldw(const T* p, float (&o)[VW]) {
+  if constexpr (VW == 8) {
+    ld8(p, o);
+  } else if constexpr (sizeof(T) == 2) {
+    const uint2 v = *reinterpret_cast<const uint2*>(p);
+    o[0] = bflo(v.x); o[1] = bfhi(v.x); o[2] = bflo(v.y); o[3] = bfhi(v.y);
+  } else {
+    const float4 v = *reinterpret_cast<const float4*>(p);
+    o[0] = v.x; o[1] = v.y; o[2] = v.z; o[3] = v.w;
+  }
+}
+template <int VW, typename T>
+__device__ __forceinline__ void stw(T* p, const float (&v)[VW]) {
+  if constexpr (VW == 8) st8(p, v);
+  else if constexpr (sizeof(T) == 2) *reinterpret_cast<uint2*>(p) = make_uint2(pack2bf(v[0], v[1]), pack2bf(v[2], v[3]));
+  else *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+}
+
+// One workgroup of NT threads per row, VW columns per thread and step, widths up to VW * NT * NV held in registers. Many
+// rows: 256 threads of 8 columns; few rows (decode steps): 1024 of 4, a row's loads spread over more waves.
+template <typename T, int S, int NV, int NT, int VW>
+__global__ __launch_bounds__(NT) void streams_kernel(StreamsParams p) {
+  constexpr int NW = NT / 64;
+  __shared__ float red[NW];
   const int i = blockIdx.x, tid = threadIdx.x, C = p.C;
   const size_t m = p.rows ? p.rows[i] : i;
   float* xr = p.x + m * S * p.ldx;
   const T* yr = p.tok ? (const T*)p.embed + (size_t)p.tok[m] * p.lde : (const T*)p.y + m * p.ldy;
   if (p.tok && p.pos && tid == 0) p.pos[i] += 1;
-  float u[NV][8], wv[NV][8];
+  float u[NV][VW], wv[NV][VW];
   float sum = 0.f;
 #pragma unroll
   for (int v = 0; v < NV; ++v) {
-    const int k = 8 * (tid + 256 * v);
+    const int k = VW * (tid + NT * v);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) u[v][e] = 0.f;
+    for (int e = 0; e < VW; ++e) u[v][e] = 0.f;
     if (k < C) {
-      float y[8], x[S][8];
-      ld8(yr + k, y);
-      ld8((const T*)p.w + k, wv[v]);
+      float y[VW], x[S][VW];
+      ldw<VW>(yr + k, y);
+      ldw<VW>((const T*)p.w + k, wv[v]);
       if (!p.tok) {
 #pragma unroll
-        for (int s = 0; s < S; ++s) ld8(xr + (size_t)s * p.ldx + k, x[s]);
+        for (int s = 0; s < S; ++s) ldw<VW>(xr + (size_t)s * p.ldx + k, x[s]);
       }
 #pragma unroll
       for (int t = 0; t < S; ++t) {
         const float in = p.in ? p.in[t] : 1.f;
-        float n[8];
+        float n[VW];
         if (p.tok) {
 #pragma unroll
-          for (int e = 0; e < 8; ++e) n[e] = y[e] * p.scale;
+          for (int e = 0; e < VW; ++e) n[e] = y[e] * p.scale;
         } else {
           const float ot = p.out[t];
 #pragma unroll
-          for (int e = 0; e < 8; ++e) n[e] = ot * y[e];
+          for (int e = 0; e < VW; ++e) n[e] = ot * y[e];
 #pragma unroll
           for (int s = 0; s < S; ++s) {
             const float a = p.mix[s * S + t];
 #pragma unroll
-            for (int e = 0; e < 8; ++e) n[e] += a * x[s][e];
+            for (int e = 0; e < VW; ++e) n[e] += a * x[s][e];
           }
         }
-        if (!p.rows) st8(xr + (size_t)t * p.ldx + k, n);
+        if (!p.rows) stw<VW>(xr + (size_t)t * p.ldx + k, n);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) u[v][e] += in * n[e];
+        for (int e = 0; e < VW; ++e) u[v][e] += in * n[e];
       }
 #pragma unroll
-      for (int e = 0; e < 8; ++e) sum += u[v][e];
+      for (int e = 0; e < VW; ++e) sum += u[v][e];
     }
   }
-  const float mean = block_sum4(sum, red) / (float)C;
+  const float mean = block_sum<NW>(sum, red) / (float)C;
   sum = 0.f;
 #pragma unroll
   for (int v = 0; v < NV; ++v)
-    if (8 * (tid + 256 * v) < C) {
+    if (VW * (tid + NT * v) < C) {
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
+      for (int e = 0; e < VW; ++e) {
         u[v][e] -= mean;
         sum += u[v][e] * u[v][e];
       }
     }
-  const float rs = 1.f / sqrtf(block_sum4(sum, red) / (float)C + p.eps);
+  const float rs = 1.f / sqrtf(block_sum<NW>(sum, red) / (float)C + p.eps);
   T* hr = (T*)p.h + (size_t)i * p.ldh;
 #pragma unroll
   for (int v = 0; v < NV; ++v) {
-    const int k = 8 * (tid + 256 * v);
+    const int k = VW * (tid + NT * v);
     if (k < C) {
 #pragma unroll
-      for (int e = 0; e < 8; ++e) u[v][e] *= rs * wv[v][e];
-      st8(hr + k, u[v]);
+      for (int e = 0; e < VW; ++e) u[v][e] *= rs * wv[v][e];
+      stw<VW>(hr + k, u[v]);
     }
   }
-  for (int k = C + tid; k < p.ldh; k += 256) stv(hr, k, 0.f);
+  for (int k = C + tid; k < p.ldh; k += NT) stv(hr, k, 0.f);
 }
 
 // Any width and number of streams: a column at a time, its old streams in the thread's own LDS words (so the
@@ -144,19 +171,20 @@ __global__ __launch_bounds__(256) void streams_any_kernel(StreamsParams p) {
     u[k] = a;
     sum += a;
   }
-  const float mean = block_sum4(sum, red) / (float)C;
+  const float mean = block_sum<4>(sum, red) / (float)C;
   sum = 0.f;
   for (int k = tid; k < C; k += 256) sum += (u[k] - mean) * (u[k] - mean);
-  const float rs = 1.f / sqrtf(block_sum4(sum, red) / (float)C + p.eps);
+  const float rs = 1.f / sqrtf(block_sum<4>(sum, red) / (float)C + p.eps);
   T* hr = (T*)p.h + (size_t)i * p.ldh;
   for (int k = tid; k < p.ldh; k += 256) stv(hr, k, k < C ? (u[k] - mean) * rs * ldv((const T*)p.w, k) : 0.f);
 }
 
 template <typename T, int S>
 static int streams_wide(const StreamsParams& p, int M, hipStream_t s) {
-  if (p.C <= 2048) hipLaunchKernelGGL((streams_kernel<T, S, 1>), dim3(M), dim3(256), 0, s, p);
-  else if (p.C <= 4096) hipLaunchKernelGGL((streams_kernel<T, S, 2>), dim3(M), dim3(256), 0, s, p);
-  else hipLaunchKernelGGL((streams_kernel<T, S, 4>), dim3(M), dim3(256), 0, s, p);
+  if (M <= kFewRows && p.C <= 4096) hipLaunchKernelGGL((streams_kernel<T, S, 1, 1024, 4>), dim3(M), dim3(1024), 0, s, p);
+  else if (p.C <= 2048) hipLaunchKernelGGL((streams_kernel<T, S, 1, 256, 8>), dim3(M), dim3(256), 0, s, p);
+  else if (p.C <= 4096) hipLaunchKernelGGL((streams_kernel<T, S, 2, 256, 8>), dim3(M), dim3(256), 0, s, p);
+  else hipLaunchKernelGGL((streams_kernel<T, S, 1, 1024, 8>), dim3(M), dim3(1024), 0, s, p);
   LLJ_CHECK_LAUNCH();
   return 0;
 }

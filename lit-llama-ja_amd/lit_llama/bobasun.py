@@ -70,7 +70,7 @@ class BobasunConfig:
             (factor,) = (1.0,) if scaling is None else take_values(scaling, where + ".mixer.rot.scaling", factor=float)
             if min(heads, kv, dim, vdim) < 1 or heads % kv:
                 raise ValueError(f"config: {where} has {heads} query heads on {kv} key / value heads of {dim} and {vdim}")
-            if dims % 2 or not 0 < dims <= dim:
+            if dims % 2 or not 0 <= dims <= dim:
                 raise ValueError(f"config: {where} rotates {dims} of {dim} dimensions")
             if v_mix:
                 mixing = mixing or (kv, vdim)

@@ -21,6 +21,7 @@ STREAM_ROWS = 16
 GLA_CHUNK_RANK = 240  # largest decay rank the chunked recurrence stages
 GLA_CHUNK_MIN = 16  # prompts with a sequence longer than this take the chunked recurrence
 ATTEND_WGS = 128  # latent decode attention: workgroups the visible keys of a batch are split for (one row: twice)
+STREAMS_COLUMNS = 16384  # widest product that also updates the residual streams (7B gated unit, 26112: 61 us against 46 + 4.5)
 GQA_WGS = 512  # grouped-query decode attention: workgroups the keys of a batch are split for
 GQA_RANGE = 128  # its shortest key range
 GQA_LONG = 1024  # prompts with a sequence this long take 128 queries per workgroup
@@ -123,8 +124,9 @@ class PackedLinear:
 
 
     def takes_streams(self, M: int, width: int, streams: int) -> bool:
-        """Whether apply_streams serves these rows."""
-        return (self.dtype == torch.bfloat16 and M == 1 and width == self.K and
+        """Whether apply_streams serves these rows (every workgroup of the product reads all streams: with many
+        columns a launch of their own is faster)."""
+        return (self.dtype == torch.bfloat16 and M == 1 and width == self.K and self.Np <= STREAMS_COLUMNS and
                 bool(_hip.lib().llj_streams_linear_ok(streams, width)))
 
     def apply_streams(self, y: torch.Tensor, done, x: torch.Tensor, x_out: torch.Tensor, sub, eps: float, out: torch.Tensor,

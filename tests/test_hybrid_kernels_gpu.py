@@ -1,9 +1,10 @@
-"""The hybrid models' kernels one by one (csrc/postnorm, post_gemv, gemm_bf16, gla, latent*) against
-oracle/mugivik_np.py's functions or plain float64 numpy."""
+"""The hybrid models' kernels one by one (csrc/postnorm, post_gemv, gemm_bf16, gla, latent*, streams, gqa) against
+the functions of oracle/mugivik_np.py and oracle/bobasun_np.py or plain float64 numpy."""
 import numpy as np
 import pytest
 import torch
 
+from oracle import bobasun_np as B
 from oracle import mugivik_np as O
 
 pytestmark = pytest.mark.gpu
@@ -334,3 +335,301 @@ def test_next_token_row_positions(hip, dtype):
         for r, t in enumerate(cur.tolist()):
             assert t in np.argsort(-back(lg)[r, :100], kind="stable")[:6]
     assert len(seen) > 10
+
+
+# ------------------------------------------------------------------------------------ biases and the gated unit
+def _unit_ref(y, limit, alpha):
+    g, u = np.minimum(y[:, 0::2], limit), np.clip(y[:, 1::2], -limit, limit)
+    return g * B.sigmoid(alpha * g) * (u + 1.0)
+
+
+@pytest.mark.parametrize("M", [1, 8, 9, 16, 64, 100, 256, 300, 1024])
+@pytest.mark.parametrize("N,K", [(128, 128), (2048, 1024), (384, 2048), (4352, 1152)])
+@pytest.mark.parametrize("act", [0, 2])
+def test_bias_and_unit_products(hip, M, N, K, act):
+    from lit_llama import _hip
+
+    g = torch.Generator(device="cuda").manual_seed(M + N + K)
+    A = torch.randn(M, K, generator=g, device="cuda").to(torch.bfloat16)
+    W = (torch.randn(N, K, generator=g, device="cuda") * K ** -0.5).to(torch.bfloat16)
+    bias = 2.0 * torch.randn(N, generator=g, device="cuda")
+    limit, alpha, C = 1.25, 1.5, N // 2 if act else N
+    for b in (bias, None):
+        y = back(A) @ back(W).T + (0 if b is None else back(b))
+        want = _unit_ref(y, limit, alpha) if act else y
+        out = torch.full((M, C + 16), 3.0, dtype=torch.bfloat16, device="cuda")
+        if M <= 16:
+            call("llj_rows_linear", act, A, K, W, b, out, C + 16, M, N, K, limit, alpha)
+            close(back(out)[:, :C], want, 6e-3)
+        else:
+            nb = _hip.lib().llj_gemm_bf16_ws_bytes(M, N, K)
+            for ws in {None, nb or None}:
+                buf = None if ws is None else torch.empty(nb // 4, device="cuda")
+                out.fill_(3.0)
+                call("llj_gemm_bf16", act, A, K, W, b, out, C + 16, M, N, K, limit, alpha, buf, nb)
+                close(back(out)[:, :C], want, 6e-3, ws)
+        assert float((out[:, C:] - 3.0).abs().max()) == 0.0
+
+
+@pytest.mark.parametrize("opt", [0, 100])  # LDS-DMA tiles of 256 x 128 / 256 x 256
+def test_unit_gemm_tiles(hip, opt):
+    from lit_llama import _hip
+
+    g = torch.Generator(device="cuda").manual_seed(opt)
+    M, N, K = 520, 512, 256
+    A, W = torch.randn(M, K, generator=g, device="cuda").to(torch.bfloat16), (torch.randn(N, K, generator=g, device="cuda") / 16).to(torch.bfloat16)
+    bias, y = torch.randn(N, generator=g, device="cuda"), None
+    old = _hip.lib().llj_set_option(_hip.OPT_GLDS_COST128, opt)
+    try:
+        for act, C in ((0, N), (2, N // 2)):
+            out = torch.empty(M, C, dtype=torch.bfloat16, device="cuda")
+            call("llj_gemm_bf16", act, A, K, W, bias, out, C, M, N, K, 1.0, 1.7, None, 0)
+            y = back(A) @ back(W).T + back(bias)
+            close(back(out), _unit_ref(y, 1.0, 1.7) if act else y, 6e-3, act)
+    finally:
+        _hip.lib().llj_set_option(_hip.OPT_GLDS_COST128, old)
+
+
+@pytest.mark.parametrize("dtype", list(DT))
+def test_bias_act(hip, dtype):
+    g = np.random.default_rng(3)
+    M, N, ld = 5, 42, 48
+    y, bias = dev(4 * g.standard_normal((M, ld)), dtype), dev(g.standard_normal(N))
+    rel = 2e-6 if dtype == torch.float32 else 6e-3
+    out = torch.full((M, 24), 3.0, dtype=dtype, device="cuda")
+    for b in (bias, None):
+        call("llj_g_bias_act", 2, y, ld, b, out, 24, M, N, 1.5, 1.7, DT[dtype])
+        close(back(out)[:, :21], _unit_ref(back(y)[:, :N] + (0 if b is None else back(b)), 1.5, 1.7), rel)
+    y0 = back(y)
+    call("llj_g_bias_act", 0, y, ld, bias, None, 0, M, N, 0.0, 0.0, DT[dtype])
+    close(back(y)[:, :N], y0[:, :N] + back(bias), rel)
+    assert (back(y)[:, N:] == y0[:, N:]).all() and float((out[:, 21:] - 3.0).abs().max()) == 0.0
+
+
+# ------------------------------------------------------------------------------------ residual streams
+def _streams_case(g, M, S, C, ld, dtype):
+    hc = {"in": dev(g.standard_normal(S)), "out": dev(g.standard_normal(S)), "mix": dev(g.standard_normal((S, S)))}
+    x, y = dev(3 + g.standard_normal((M, S, ld))), dev(2 * g.standard_normal((M, ld)), dtype)
+    return hc, {k: back(v) for k, v in hc.items()}, x, y, dev(1 + 0.3 * g.standard_normal(C), dtype)
+
+
+@pytest.mark.parametrize("dtype", list(DT))
+@pytest.mark.parametrize("M", [3, 70])
+@pytest.mark.parametrize("S,C", [(1, 8), (2, 72), (3, 75), (4, 2048), (3, 4096), (5, 320), (4, 5120), (2, 8192), (2, 9000), (9, 64)])
+def test_streams_step(hip, dtype, M, S, C):
+    g = np.random.default_rng(C + S)
+    ld, eps = (C + 7) // 8 * 8 + 8, 1e-5
+    hc, ref, x, y, w = _streams_case(g, M, S, C, ld, dtype)
+    X = back(x)[..., :C].transpose(1, 0, 2)
+    new = B.streams_out(X, back(y)[:, :C], ref)
+    rel = 3e-6 if dtype == torch.float32 else 6e-3
+    x0 = x.clone()
+    pick = ints(2, 0)
+    h = torch.full((M, ld), 7.0, dtype=dtype, device="cuda")
+    call("llj_streams_step", y, ld, hc["out"], hc["mix"], x, ld, S, None, w, eps, h, ld, pick, 2, C, DT[dtype])
+    assert torch.equal(x, x0)
+    close(back(h)[:2, :C], B.layer_norm(new.sum(0), back(w), eps)[[2, 0]], rel, "gathered sum")
+    call("llj_streams_step", y, ld, hc["out"], hc["mix"], x, ld, S, hc["in"], w, eps, h, ld, None, M, C, DT[dtype])
+    close(back(x)[..., :C].transpose(1, 0, 2), new, 2e-6, "streams")
+    close(back(h)[:, :C], B.layer_norm(B.streams_in(new, ref), back(w), eps), rel, "normed")
+    assert float(h[:, C:].abs().max()) == 0.0 and torch.equal(x[..., C:], x0[..., C:])
+
+
+@pytest.mark.parametrize("dtype", list(DT))
+@pytest.mark.parametrize("S,C", [(2, 72), (3, 75), (4, 2048), (7, 40)])
+def test_streams_embed(hip, dtype, S, C):
+    g = np.random.default_rng(S)
+    emb, tok = dev(g.standard_normal((11, C)), dtype), ints(3, 10, 0, 3)
+    hc, ref, x, _, w = _streams_case(g, 4, S, C, C, dtype)
+    h, pos = torch.empty(4, C, dtype=dtype, device="cuda"), ints(5, 0, 2, 9)
+    e = back(emb)[[3, 10, 0, 3]] * 1.5
+    for ps in (pos, None):
+        call("llj_streams_embed", tok, emb, C, 1.5, ps, x, C, S, hc["in"], w, 1e-6, h, C, 4, C, DT[dtype])
+        close(back(x), np.stack([e] * S, 1), 1e-6)
+        close(back(h), B.layer_norm(ref["in"].sum() * e, back(w), 1e-6), 1e-5 if dtype == torch.float32 else 6e-3)
+    assert pos.tolist() == [6, 1, 3, 10]
+
+
+@pytest.mark.parametrize("S,C,K,N", [(1, 72, 128, 256), (2, 2048, 2048, 384), (4, 4096, 4096, 128), (3, 8192, 8192, 4224),
+                                     (4, 1000, 1024, 8448)])
+@pytest.mark.parametrize("act", [0, 2])
+def test_streams_linear(hip, S, C, K, N, act):
+    g = np.random.default_rng(C + N)
+    hc, ref, x, y, w = _streams_case(g, 1, S, C, C, torch.bfloat16)
+    W, bias = dev(g.standard_normal((N, K)) * C ** -0.5, torch.bfloat16), dev(g.standard_normal(N))
+    xo, out = torch.zeros_like(x), torch.empty(N // 2 if act else N, dtype=torch.bfloat16, device="cuda")
+    call("llj_streams_linear", act, y, hc["out"], hc["mix"], x, xo, C, S, hc["in"], w, 1e-5, C, W, bias, out, N, K, 1.25, 1.5)
+    new = B.streams_out(back(x).transpose(1, 0, 2), back(y), ref)
+    close(back(xo).transpose(1, 0, 2), new, 2e-6)
+    v = B.layer_norm(B.streams_in(new, ref), back(w), 1e-5) @ back(W)[:, :C].T + back(bias)
+    close(back(out), _unit_ref(v, 1.25, 1.5)[0] if act else v[0], 1.2e-2)
+
+
+# ------------------------------------------------------------------------------------ grouped-query attention
+class GqaCase:
+    """Packed projections of sequences that go on from `starts` cached tokens, and the float64 reference."""
+
+    def __init__(self, seed, H, G, D, V, RD, starts, lens, dtype, norm=1, sink=1, scale=None, vmode=0, gate=True, plant=None):
+        g = np.random.default_rng(seed)
+        self.H, self.G, self.D, self.V, self.RD, self.dtype, self.norm, self.sink = H, G, D, V, RD, dtype, norm, sink
+        self.starts, self.lens, self.M, self.vmode = starts, lens, sum(lens), vmode
+        self.scale = D ** -0.5 if scale is None else scale
+        up = lambda n: (n + 7) // 8 * 8  # noqa: E731
+        self.o = [0, up(H * D), up(H * D) + up(G * D), up(H * D) + up(G * D) + up(G * V)]
+        self.ld, self.W, self.ldc = up(self.o[3] + H), max(a + b for a, b in zip(starts, lens)) + 3, up(G * (D + V))
+        self.eps, self.base, self.factor = 1e-5, 70.0, 1.5
+        self.inp = dev(1.5 * g.standard_normal((self.M, self.ld)), dtype)
+        self.slots = list(g.permutation(len(lens) + 2)[:len(lens)])
+        self.cache = dev(g.standard_normal((len(lens) + 2, self.W, self.ldc)), dtype)
+        if plant is not None:  # every query and one key per sequence share a direction
+            q, c = back(self.inp), back(self.cache)
+            q[:, :H * D].reshape(self.M, H, D)[:, :, -1] = 6.0
+            q[:, self.o[1]:self.o[1] + G * D].reshape(self.M, G, D)[:, :, -1] = 0.0
+            c[:, :, :G * D].reshape(-1, self.W, G, D)[..., -1] = 0.0
+            row = 0
+            for s, n, sl in zip(starts, lens, self.slots):
+                if plant < s:
+                    c[sl, plant, :G * D].reshape(G, D)[:, -1] = 6.0
+                elif plant < s + n:
+                    q[row + plant - s, self.o[1]:self.o[1] + G * D].reshape(G, D)[:, -1] = 6.0
+                row += n
+            self.inp, self.cache = dev(q, dtype), dev(c, dtype)
+        self.lam, self.first = dev([0.3]), dev(g.standard_normal((self.M, G * V)), dtype)
+        self.gate = gate
+        i = torch.arange(0, RD, 2, dtype=torch.float64)
+        self.turns = (self.base ** (-i / max(RD, 1)) / self.factor / (2 * np.pi)).cuda()
+        self.pos = ints(*[s + j for s, n in zip(starts, lens) for j in range(n)])
+        self.seq = ints(*[b for b, n in enumerate(lens) for _ in range(n)])
+        self.slot = ints(*self.slots)
+        self.args = (self.M, H, G, D, V)
+
+    def reference(self):
+        """(outputs, cache after, first after)"""
+        H, G, D, V, o = self.H, self.G, self.D, self.V, self.o
+        p, cache, first = back(self.inp), back(self.cache), back(self.first)
+        pos = np.array(self.pos.tolist())
+        def prep(t):
+            t = B.rotate_half(t, pos, self.base, self.RD, self.factor) if self.RD else t
+            return B.unit_rms(t, self.eps) if self.norm else t
+        q, k = prep(p[:, :H * D].reshape(-1, H, D)), prep(p[:, o[1]:o[1] + G * D].reshape(-1, G, D))
+        v = p[:, o[2]:o[2] + G * V]
+        if self.vmode == 1:
+            first = v.copy()
+        elif self.vmode == 2:
+            v = B.mix_values(v, first, float(back(self.lam)[0]))
+        y, row = np.empty((self.M, H * V)), 0
+        for s, n, sl in zip(self.starts, self.lens, self.slots):
+            r = slice(row, row + n)
+            cache[sl, s:s + n, :G * D], cache[sl, s:s + n, G * D:G * (D + V)] = k[r].reshape(n, -1), v[r]
+            K, Vv = cache[sl, :s + n, :G * D].reshape(-1, G, D), cache[sl, :s + n, G * D:G * (D + V)].reshape(-1, G, V)
+            for i in range(n):
+                for h in range(H):
+                    gh, e = h // (H // G), s + i + 1
+                    sc = K[:e, gh] @ q[row + i, h] * self.scale
+                    m = max(sc.max(), 0.0) if self.sink else sc.max()
+                    w = np.exp(sc - m)
+                    out = w @ Vv[:e, gh] / (w.sum() + (np.exp(-m) if self.sink else 0.0))
+                    y[row + i, h * V:(h + 1) * V] = out * (B.sigmoid(p[row + i, o[3] + h]) if self.gate else 1.0)
+            row += n
+        return y, cache, first
+
+    def new(self):
+        """arguments for the rows' own keys and values"""
+        first = self.first if self.vmode else None
+        return (self.pos,), (self.turns, self.RD, self.norm, self.eps), (first, self.lam if self.vmode == 2 else None, self.G * self.V)
+
+    def og(self):
+        return self.o[3] if self.gate else -1
+
+    def verify(self, y, what=""):
+        want, cache, first = self.want
+        f32 = self.dtype == torch.float32
+        close(back(y)[:, :self.H * self.V], want, 5e-6 if f32 else 2e-2, what)
+        n = self.G * (self.D + self.V)
+        close(back(self.cache)[..., :n], cache[..., :n], 3e-6 if f32 else 8e-3, f"{what} cache")
+        close(back(self.first), first, 1e-7, f"{what} first values")
+
+    def run(self, kind):
+        self.want = self.reference()
+        y = torch.zeros(self.M, (self.H * self.V + 7) // 8 * 8, dtype=self.dtype, device="cuda")
+        o, dt = self.o, DT[self.dtype]
+        (pos,), rot, mixed = self.new()
+        if kind == "decode":
+            from lit_llama import _hip
+
+            for n in (1, 2, 7):
+                part = torch.full((self.M * self.H * n * _hip.lib().llj_gqa_part_width(self.V),), 9.0, device="cuda")
+                call("llj_gqa_decode", self.inp, self.ld, *o[:3], self.og(), *rot, pos, self.slot, self.cache, self.W, self.ldc,
+                     *mixed, part, n, y, y.stride(0), *self.args, self.scale, self.sink)
+                self.verify(y, n)
+            return
+        call("llj_gqa_prep", self.inp, self.ld, *o[:3], *rot, pos, self.seq, self.slot, self.cache, self.W, self.ldc, *mixed,
+             *self.args, dt)
+        if kind == "rows":
+            call("llj_gqa_rows", self.inp, self.ld, o[0], self.og(), pos, self.seq, self.slot, self.cache, self.W, self.ldc, y,
+                 y.stride(0), *self.args, self.scale, self.sink, dt)
+        else:
+            from lit_llama.state import Rows
+
+            r = Rows.packed([[0] * n for n in self.lens], self.starts, [int(s) for s in self.slots], "cuda")
+            n, work = r.pairs(kind)
+            call("llj_gqa_flash", self.inp, self.ld, o[0], self.og(), work, n, kind, pos, self.slot, self.cache, self.W, self.ldc, y,
+                 y.stride(0), *self.args, self.scale, self.sink)
+        self.verify(y, kind)
+
+
+GQA_SIZES = [(3, 1, 10, 14, 6), (4, 2, 7, 5, 0), (2, 2, 1, 1, 0), (6, 2, 48, 24, 16), (8, 1, 128, 128, 128), (20, 1, 96, 64, 64),
+             (2, 1, 256, 168, 32), (40, 2, 64, 96, 64), (1, 1, 600, 300, 320)]
+
+
+@pytest.mark.parametrize("dtype", list(DT))
+@pytest.mark.parametrize("H,G,D,V,RD", GQA_SIZES)
+@pytest.mark.parametrize("vmode", [0, 1, 2])
+def test_gqa_rows(hip, dtype, H, G, D, V, RD, vmode):
+    GqaCase(D + vmode, H, G, D, V, RD, [0, 40, 300], [5, 1, 3], dtype, vmode=vmode).run("rows")
+
+
+@pytest.mark.parametrize("H,G,D,V,RD", [s for s in GQA_SIZES if s[2] % 8 == 0 and s[3] % 8 == 0 and s[2] <= 256])
+@pytest.mark.parametrize("rows", [64, 128])
+def test_gqa_flash(hip, H, G, D, V, RD, rows):
+    if rows == 128 and max(D, V) > 128:
+        pytest.skip("64-query blocks only")
+    GqaCase(D, H, G, D, V, RD, [0, 40, 0], [70, 130, 200], torch.bfloat16, vmode=2).run(rows)
+
+
+@pytest.mark.parametrize("H,G,D,V,RD", [s for s in GQA_SIZES if s[2] % 8 == 0 and s[3] % 8 == 0 and s[2] <= 256])
+@pytest.mark.parametrize("vmode", [0, 1, 2])
+def test_gqa_decode(hip, H, G, D, V, RD, vmode):
+    GqaCase(D + vmode, H, G, D, V, RD, [0, 1, 31, 32, 33, 127, 128, 500], [1] * 8, torch.bfloat16, vmode=vmode).run("decode")
+
+
+@pytest.mark.parametrize("kind,dtype", [("rows", torch.float32), ("rows", torch.bfloat16), (64, torch.bfloat16), (128, torch.bfloat16),
+                                        ("decode", torch.bfloat16)])
+@pytest.mark.parametrize("option", [dict(norm=0), dict(sink=0), dict(gate=False), dict(norm=0, scale=-0.2), dict(scale=1.5),
+                                    dict(norm=0, scale=0.6), dict(norm=0, scale=0.6, sink=0)])
+def test_gqa_options(hip, kind, dtype, option):
+    lens = [1] * 3 if kind == "decode" else [66, 3, 90]
+    GqaCase(5, 6, 2, 48, 24, 32, [0, 90, 33], lens, dtype, **option).run(kind)
+
+
+@pytest.mark.parametrize("kind,dtype", [("rows", torch.float32), (64, torch.bfloat16), (128, torch.bfloat16), ("decode", torch.bfloat16)])
+@pytest.mark.parametrize("key", [0, 1, 15, 16, 31, 32, 63, 64, 95, 96, 127, 128, 199, 200])
+def test_gqa_one_key_stands_out(hip, kind, dtype, key):
+    """Each query's weight lies almost wholly on one key (its own, or one at a tile's edge): the output is that value."""
+    starts, lens = ([200, key, 230], [1, 1, 1]) if kind == "decode" else ([0, key, 100], [202, 4, 105])
+    c = GqaCase(key, 4, 2, 32, 16, 16, starts, lens, dtype, norm=0, scale=0.5, plant=key)
+    c.run(kind)
+
+
+@pytest.mark.parametrize("kind,dtype", [("rows", torch.float32), (64, torch.bfloat16), ("decode", torch.bfloat16)])
+def test_gqa_sink_takes_the_weight(hip, kind, dtype):
+    """Scores far below 0 leave the weight to the sink: the outputs almost vanish, and would be averages without it."""
+    lens = [1] * 2 if kind == "decode" else [70, 9]
+    c = GqaCase(1, 2, 1, 32, 16, 0, [0, 64], lens, dtype, norm=0, scale=1.0, gate=False)
+    q, k = back(c.inp), back(c.cache)
+    q[:, :64] = 1.0
+    q[:, c.o[1]:c.o[1] + 32] = -0.2
+    k[..., :32] = -0.2
+    c.inp, c.cache = dev(q, dtype), dev(k, dtype)
+    c.run(kind)
+    assert np.abs(c.want[0]).max() < 0.15
