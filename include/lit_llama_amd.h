@@ -515,8 +515,9 @@ int llj_streams_linear(int act, const void* y, const float* out_w, const float* 
  * denominator; y = sum p v * sigmoid(gate).
  * flash: prompt rows (bf16, MFMA); work = two (first row, rows, sequence) blocks of at most `rows` rows each per entry (the
  * second's rows 0: none), rows = llj_gqa_flash_rows (0: not these sizes).
- * decode: one row per sequence (bf16, MFMA), prep included; part [M][heads][nsplit][llj_gqa_part_width(vdim)] fp32 scratch,
- * nsplit <= 64 key ranges. */
+ * decode: one row per sequence (bf16, MFMA), prep included, nsplit <= 64 key ranges; scratch part
+ * [M][heads][nsplit][llj_gqa_part_width(vdim)] fp32 and count [M][heads] ints, zero before the first call (a call leaves
+ * them zero). */
 int llj_gqa_prep(void* in, int ld, int oq, int ok, int ov, const void* turns, int rot_dims, int qk_norm, float eps,
                  const int* pos, const int* row_seq, const int* slot, void* cache, int W, int ldc, void* first,
                  const float* lam, int ldf, int M, int heads, int kv_heads, int dim, int vdim, int dt, void* stream);
@@ -531,7 +532,7 @@ int llj_gqa_decode_ok(int dim, int vdim);
 int llj_gqa_part_width(int vdim);
 int llj_gqa_decode(const void* in, int ld, int oq, int ok, int ov, int og, const void* turns, int rot_dims, int qk_norm,
                    float eps, const int* pos, const int* slot, void* cache, int W, int ldc, void* first, const float* lam,
-                   int ldf, float* part, int nsplit, void* y, int ldy, int M, int heads, int kv_heads, int dim, int vdim,
+                   int ldf, float* part, int* count, int nsplit, void* y, int ldy, int M, int heads, int kv_heads, int dim, int vdim,
                    float scale, int sink, void* stream);
 
 /* Measurement aid (no reference counterpart): reads `bytes` (a multiple of 16) at p once with

@@ -37,6 +37,16 @@ struct GqaParams {
   float scale;
 };
 
+// device-scope accesses of the decode hand-off, two floats each
+__device__ __forceinline__ void put2(float* p, float a, float b) {
+  const unsigned long long v = (unsigned long long)__float_as_uint(a) | ((unsigned long long)__float_as_uint(b) << 32);
+  __hip_atomic_store(reinterpret_cast<unsigned long long*>(p), v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+}
+__device__ __forceinline__ float2 get2(const float* p) {
+  const unsigned long long v = __hip_atomic_load(reinterpret_cast<const unsigned long long*>(p), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  return make_float2(__uint_as_float((uint32_t)v), __uint_as_float((uint32_t)(v >> 32)));
+}
+
 __device__ __forceinline__ void turn_cs(const double* __restrict__ turns, int i, int pos, float& c, float& s) {
   const double t = (double)pos * turns[i];
   sincospif(2.f * (float)(t - rint(t)), &s, &c);
@@ -370,13 +380,15 @@ __global__ __launch_bounds__(256, 2) void gqa_flash_kernel(GqaParams p, const in
 // them in the cache and takes them from LDS. The waves then walk 32-key steps of the range on their own (no
 // barriers): K fragments straight from the cache, S^T = K q^T, P from the accumulators, V through a wave's LDS
 // tile and transposing reads. The waves' results are merged through LDS; one range: the result itself, else fp32 partials
-// [M][H][nsplit][VW + 4] (o unnormalized, then max in log2 units, sum) for the combine kernel.
+// [M][H][nsplit][VW + 4] (o unnormalized, then max in log2 units, sum), which the last of the ranges' workgroups to
+// finish merges in range order. The hand-off: device-scope (write-through) stores, a wait for them, one device-scope
+// counter per (row, heads), device-scope loads; nobody waits for another workgroup, and the last one resets the counter.
 __host__ __device__ constexpr size_t gqa_attend_lds(int KT, int DB, int n) {
   return (size_t)(17 * (KT * 32 + 8) + DB * 16) * 2 + (size_t)4 * 32 * (DB * 16 + 16) * 2 + (size_t)2 * n * 4 + 2 * 64 * 4;
 }
 
 template <int KT, int DB>
-__global__ __launch_bounds__(256) void gqa_attend_kernel(GqaParams p, float* __restrict__ partials, int nsplit, float sl2) {
+__global__ __launch_bounds__(256) void gqa_attend_kernel(GqaParams p, float* partials, int* count, int nsplit, float sl2) {
   constexpr int KW = KT * 32, QP = KW + 8, VW = DB * 16, VP = VW + 16;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   bf16_t* Qs = reinterpret_cast<bf16_t*>(smem);  // [16][QP] queries, then the new key
@@ -627,41 +639,60 @@ __global__ __launch_bounds__(256) void gqa_attend_kernel(GqaParams p, float* __r
       if (v < V) *reinterpret_cast<uint2*>(yr) = make_uint2(pack2bf(o[0] * f, o[1] * f), pack2bf(o[2] * f, o[3] * f));
     } else {
       float* dst = partials + (((size_t)m * p.H + h0 + hh) * nsplit + sp) * RP;
-      *reinterpret_cast<f32x4*>(dst + v) = o;
-      if (v == 0) {
-        dst[VW] = mx;
-        dst[VW + 1] = l;
-      }
+      put2(dst + v, o[0], o[1]);
+      put2(dst + v + 2, o[2], o[3]);
+      if (v == 0) put2(dst + VW, mx, l);
     }
   }
-}
-
-// the ranges of one (head, row) merged in order, the sink, the gate; VW / 4 lanes per 4-column piece, 4 waves over the
-// ranges
-__global__ __launch_bounds__(256) void gqa_combine_kernel(GqaParams p, const float* __restrict__ partials, int nsplit, int VW) {
-  __shared__ float sw[64];
-  __shared__ f32x4 red[4][64];
-  const int h = blockIdx.x, m = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = uniform(tid >> 6);
-  const int RP = VW + 4, v = 4 * lane;
-  const float* part = partials + ((size_t)m * p.H + h) * nsplit * RP;
-  const float gate = p.og >= 0 ? bf2f(((const bf16_t*)p.in)[(size_t)m * p.ld + p.og + h]) : 0.f;
-  const float ms = lane < nsplit ? part[(size_t)lane * RP + VW] : -INFINITY;
-  const float ls = lane < nsplit ? part[(size_t)lane * RP + VW + 1] : 0.f;
-  const float mt = fmaxf(wave_max(ms), p.sink ? 0.f : -INFINITY);
-  const float w = __builtin_amdgcn_exp2f(ms - mt);
-  const float L = wave_sum(w * ls) + (p.sink ? __builtin_amdgcn_exp2f(-mt) : 0.f);
-  if (wave == 0) sw[lane] = w / L;
+  if (nsplit == 1) return;
+  // ---- the last of the ranges' workgroups merges them
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's partials are out
   __syncthreads();
-  f32x4 o = {0.f, 0.f, 0.f, 0.f};
-  if (v < VW)
-    for (int s = wave; s < nsplit; s += 4) o += *reinterpret_cast<const f32x4*>(part + (size_t)s * RP + v) * sw[s];
-  red[wave][lane] = o;
+  int* last = reinterpret_cast<int*>(wm);
+  if (tid == 0) {
+    int* c = count + (size_t)m * gridDim.y + blockIdx.y;
+    const int done = __hip_atomic_fetch_add(c, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    *last = done == nsplit - 1;
+    if (done == nsplit - 1) __hip_atomic_store(c, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
   __syncthreads();
-  if (wave == 0 && v < p.V) {
-    o = red[0][lane] + red[1][lane] + red[2][lane] + red[3][lane];
-    const float f = p.og >= 0 ? 1.f / (1.f + __expf(-gate)) : 1.f;
-    *reinterpret_cast<uint2*>((bf16_t*)p.y + (size_t)m * p.ldy + h * p.V + v) =
-        make_uint2(pack2bf(o[0] * f, o[1] * f), pack2bf(o[2] * f, o[3] * f));
+  if (!*last) return;
+  const float* part = partials + ((size_t)m * p.H + h0) * nsplit * RP;
+  float* sw = red;  // [nh][64] the ranges' weights (the waves' results are used up)
+  float2 a[8], b[8];
+  auto pieces = [&](int i, int s0) {  // 4 columns of 8 ranges (past the end: a copy, dropped)
+    const float* q = part + (size_t)(i / (VW / 4)) * nsplit * RP + 4 * (i % (VW / 4));
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float* r = q + (size_t)(s0 + e < nsplit ? s0 + e : nsplit - 1) * RP;
+      a[e] = get2(r);
+      b[e] = get2(r + 2);
+    }
+  };
+  const int tot = nh * (VW / 4);
+  if (tid < tot) pieces(tid, 0);  // in flight over the weights
+  for (int hh = wave; hh < nh; hh += 4) {  // nsplit <= 64
+    float2 st = make_float2(-INFINITY, 0.f);
+    if (lane < nsplit) st = get2(part + ((size_t)hh * nsplit + lane) * RP + VW);
+    const float gate = p.og >= 0 ? bf2f(row[p.og + h0 + hh]) : 0.f;
+    const float mt = fmaxf(wave_max(st.x), p.sink ? 0.f : -INFINITY);
+    const float w = __builtin_amdgcn_exp2f(st.x - mt);
+    float L = wave_sum(w * st.y) + (p.sink ? __builtin_amdgcn_exp2f(-mt) : 0.f);
+    if (p.og >= 0) L *= 1.f + __expf(-gate);
+    if (lane < nsplit) sw[hh * 64 + lane] = w / L;
+  }
+  __syncthreads();
+  for (int i = tid; i < tot; i += 256) {
+    const int hh = i / (VW / 4), v = 4 * (i % (VW / 4));
+    f32x4 o = {0.f, 0.f, 0.f, 0.f};
+    for (int s0 = 0; s0 < nsplit; s0 += 8) {
+      if (i != tid || s0) pieces(i, s0);
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        if (s0 + e < nsplit) o += f32x4{a[e].x, a[e].y, b[e].x, b[e].y} * sw[hh * 64 + s0 + e];
+    }
+    bf16_t* yr = (bf16_t*)p.y + (size_t)m * p.ldy + (h0 + hh) * V + v;
+    if (v < V) *reinterpret_cast<uint2*>(yr) = make_uint2(pack2bf(o[0], o[1]), pack2bf(o[2], o[3]));
   }
 }
 
@@ -702,7 +733,7 @@ static int gqa_flash_go(const GqaParams& p, const int* work, int nwork, float sl
 }
 
 template <int KT, int DB>
-static int gqa_attend_go(const GqaParams& p, float* part, int nsplit, float sl2, hipStream_t s) {
+static int gqa_attend_go(const GqaParams& p, float* part, int* count, int nsplit, float sl2, hipStream_t s) {
   auto kern = gqa_attend_kernel<KT, DB>;
   const size_t lds = gqa_attend_lds(KT, DB, p.RD / 2);
   static bool set = false;
@@ -711,9 +742,7 @@ static int gqa_attend_go(const GqaParams& p, float* part, int nsplit, float sl2,
     set = true;
   }
   const int R = p.H / p.G;
-  hipLaunchKernelGGL(kern, dim3(nsplit, p.G * ((R + 15) / 16), p.M), dim3(256), lds, s, p, part, nsplit, sl2);
-  LLJ_CHECK_LAUNCH();
-  if (nsplit > 1) hipLaunchKernelGGL(gqa_combine_kernel, dim3(p.H, p.M), dim3(256), 0, s, p, (const float*)part, nsplit, DB * 16);
+  hipLaunchKernelGGL(kern, dim3(nsplit, p.G * ((R + 15) / 16), p.M), dim3(256), lds, s, p, part, count, nsplit, sl2);
   LLJ_CHECK_LAUNCH();
   return 0;
 }
@@ -729,10 +758,10 @@ static int gqa_flash_keys(const GqaParams& p, const int* work, int nwork, int ro
 }
 
 template <int DB>
-static int gqa_attend_keys(const GqaParams& p, float* part, int nsplit, float sl2, hipStream_t s) {
-  if (p.D <= 64) return gqa_attend_go<2, DB>(p, part, nsplit, sl2, s);
-  if (p.D <= 128) return gqa_attend_go<4, DB>(p, part, nsplit, sl2, s);
-  return gqa_attend_go<8, DB>(p, part, nsplit, sl2, s);
+static int gqa_attend_keys(const GqaParams& p, float* part, int* count, int nsplit, float sl2, hipStream_t s) {
+  if (p.D <= 64) return gqa_attend_go<2, DB>(p, part, count, nsplit, sl2, s);
+  if (p.D <= 128) return gqa_attend_go<4, DB>(p, part, count, nsplit, sl2, s);
+  return gqa_attend_go<8, DB>(p, part, count, nsplit, sl2, s);
 }
 
 }  // namespace llj
@@ -818,7 +847,7 @@ int llj_gqa_part_width(int vdim) { return (vdim <= 64 ? 64 : vdim <= 128 ? 128 :
 
 int llj_gqa_decode(const void* in, int ld, int oq, int ok, int ov, int og, const void* turns, int rot_dims, int qk_norm,
                    float eps, const int* pos, const int* slot, void* cache, int W, int ldc, void* first, const float* lam,
-                   int ldf, float* part, int nsplit, void* y, int ldy, int M, int heads, int kv_heads, int dim, int vdim,
+                   int ldf, float* part, int* count, int nsplit, void* y, int ldy, int M, int heads, int kv_heads, int dim, int vdim,
                    float scale, int sink, void* stream) {
   GqaParams p{};
   p.in = (void*)in; p.ld = ld; p.oq = oq; p.ok = ok; p.ov = ov; p.og = og;
@@ -828,13 +857,13 @@ int llj_gqa_decode(const void* in, int ld, int oq, int ok, int ov, int og, const
   if (const int rc = gqa_check(p)) return rc;
   if (const int rc = gqa_check_new(p)) return rc;
   LLJ_REQUIRE(y && ldy >= heads * vdim && ldy % 4 == 0 && gqa_aligned(p) && M <= 65535 && nsplit >= 1 && nsplit <= 64 &&
-              kv_heads * ((heads / kv_heads + 15) / 16) <= 65535 && (nsplit == 1 || part) &&
+              kv_heads * ((heads / kv_heads + 15) / 16) <= 65535 && (nsplit == 1 || (part && count)) &&
               (((uintptr_t)part | (uintptr_t)y) & 15) == 0);
   const float sl2 = scale * 1.4426950408889634f;
   hipStream_t s = (hipStream_t)stream;
-  if (vdim <= 64) return gqa_attend_keys<4>(p, part, nsplit, sl2, s);
-  if (vdim <= 128) return gqa_attend_keys<8>(p, part, nsplit, sl2, s);
-  return gqa_attend_keys<16>(p, part, nsplit, sl2, s);
+  if (vdim <= 64) return gqa_attend_keys<4>(p, part, count, nsplit, sl2, s);
+  if (vdim <= 128) return gqa_attend_keys<8>(p, part, count, nsplit, sl2, s);
+  return gqa_attend_keys<16>(p, part, count, nsplit, sl2, s);
 }
 
 }  // extern "C"

@@ -118,7 +118,7 @@ SIGNATURES = {
     "llj_gqa_flash": [_P, _I, _I, _I, _P, _I, _I, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _F, _I, _P],
     "llj_gqa_decode_ok": [_I, _I],
     "llj_gqa_part_width": [_I],
-    "llj_gqa_decode": [_P, _I, _I, _I, _I, _I, _P, _I, _I, _F, _P, _P, _P, _I, _I, _P, _P, _I, _P, _I, _P, _I, _I,
+    "llj_gqa_decode": [_P, _I, _I, _I, _I, _I, _P, _I, _I, _F, _P, _P, _P, _I, _I, _P, _P, _I, _P, _P, _I, _P, _I, _I,
                        _I, _I, _I, _I, _F, _I, _P],
     "llj_g_i8_linear": [_P, _I, _I, _I, _P, _P, _F, _P, _I, _P, _I, _P, _I, _I, _P],
 }

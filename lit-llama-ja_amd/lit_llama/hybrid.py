@@ -57,11 +57,11 @@ class Scratch:
             self.hb = torch.empty(n, width, dtype=dtype, device=self.device)
         return self.hb
 
-    def buffer(self, name: str, numel: int, dtype) -> torch.Tensor:
-        """Scratch shared by the layers, at least numel long."""
+    def buffer(self, name: str, numel: int, dtype, zero: bool = False) -> torch.Tensor:
+        """Scratch shared by the layers, at least numel long; zero: cleared when it is made."""
         t = self._buffers.get(name)
         if t is None or t.numel() < numel:
-            t = self._buffers[name] = torch.empty(numel, dtype=dtype, device=self.device)
+            t = self._buffers[name] = (torch.zeros if zero else torch.empty)(numel, dtype=dtype, device=self.device)
         return t
 
 

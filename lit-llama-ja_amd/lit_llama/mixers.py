@@ -24,7 +24,8 @@ ATTEND_WGS = 128  # latent decode attention: workgroups the visible keys of a ba
 STREAMS_COLUMNS = 16384  # widest product that also updates the residual streams (7B gated unit, 26112: 61 us against 46 + 4.5)
 GQA_WGS = 512  # grouped-query decode attention: workgroups the keys of a batch are split for
 GQA_RANGE = 128  # its shortest key range
-GQA_LONG = 1024  # prompts with a sequence this long take 128 queries per workgroup
+GQA_LONG = 1024  # prompts with a sequence this long take 128 queries per workgroup where that leaves at least
+GQA_WIDE_WGS = 256  # this many workgroups
 PART_ALIGN = 8  # output columns of the parts of a packed group start at multiples of this
 
 
@@ -434,11 +435,16 @@ class GroupedAttention:
         """Key ranges of a decode step over a cache of W rows (None: the most there can be)."""
         s = self.spec
         most = max(1, min(64, GQA_WGS // (M * s.kv_heads * ((s.heads // s.kv_heads + 15) // 16))))
-        return most if W is None else max(1, min(most, (W + GQA_RANGE - 1) // GQA_RANGE))
+        if W is None:
+            return most
+        n = -(-W // GQA_RANGE)
+        return min(most, n if n <= 8 else max(8, -(-W // (2 * GQA_RANGE))))
 
     def _part(self, w, M: int, n: int):
+        """Partials and counters of a decode step's key ranges (the counters start at zero, and every step leaves them so)."""
         s = self.spec
-        return w.buffer("part", M * s.heads * n * _hip.lib().llj_gqa_part_width(s.vdim), torch.float32)
+        return (w.buffer("part", M * s.heads * n * _hip.lib().llj_gqa_part_width(s.vdim), torch.float32),
+                w.buffer("count", M * s.heads, torch.int32, zero=True))
 
     def reserve(self, w, M: int) -> None:
         if self._decode_ok():
@@ -455,14 +461,15 @@ class GroupedAttention:
         if rows.decode and self._decode_ok():
             n = self._splits(M, W)
             _hip.call("llj_gqa_decode", p.data_ptr(), p.stride(0), o[0], o[1], o[2], o[3], *new, rows.pos.data_ptr(),
-                      rows.slot.data_ptr(), cache.data_ptr(), W, ldc, *mixed, self._part(w, M, n).data_ptr(), n,
+                      rows.slot.data_ptr(), cache.data_ptr(), W, ldc, *mixed, *(t.data_ptr() for t in self._part(w, M, n)), n,
                       y.data_ptr(), y.stride(0), *sizes, s.scale, int(s.sink), st)
             return
         _hip.call("llj_gqa_prep", p.data_ptr(), p.stride(0), o[0], o[1], o[2], *new, rows.pos.data_ptr(),
                   _hip.ptr(rows.row_seq), rows.slot.data_ptr(), cache.data_ptr(), W, ldc, *mixed, *sizes, _dt(self.dtype), st)
         C = 0
         if not rows.decode and self.dtype == torch.bfloat16:
-            C = _hip.lib().llj_gqa_flash_rows(s.dim, s.vdim, int(max(rows.lengths) >= GQA_LONG))
+            wide = s.heads * sum(-(-n // 256) for n in rows.lengths)  # workgroups of two 128-query blocks
+            C = _hip.lib().llj_gqa_flash_rows(s.dim, s.vdim, int(max(rows.lengths) >= GQA_LONG and wide >= GQA_WIDE_WGS))
         if C:
             n, work = rows.pairs(C)
             _hip.call("llj_gqa_flash", p.data_ptr(), p.stride(0), o[0], o[3], work.data_ptr(), n, C, rows.pos.data_ptr(),

@@ -37,8 +37,12 @@ def test_whole_prompts(hip, name, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_long_prompt(hip, dtype):
-    """Long enough for the wider query blocks, several tiles of keys and the split products."""
+@pytest.mark.parametrize("wide", [1, 256])
+def test_long_prompt(hip, monkeypatch, dtype, wide):
+    """Long prompts in both query block sizes, several tiles of keys and the split products."""
+    from lit_llama import mixers
+
+    monkeypatch.setattr(mixers, "GQA_WIDE_WGS", wide)
     cfg, w, m = case("tiled", dtype)
     toks = prompts(cfg, [1100], seed=21)[0]
     st = m.new_state(1)

@@ -557,11 +557,13 @@ class GqaCase:
         if kind == "decode":
             from lit_llama import _hip
 
-            for n in (1, 2, 7):
+            count = torch.zeros(self.M * self.H, dtype=torch.int32, device="cuda")
+            for n in (1, 2, 7, 16):
                 part = torch.full((self.M * self.H * n * _hip.lib().llj_gqa_part_width(self.V),), 9.0, device="cuda")
                 call("llj_gqa_decode", self.inp, self.ld, *o[:3], self.og(), *rot, pos, self.slot, self.cache, self.W, self.ldc,
-                     *mixed, part, n, y, y.stride(0), *self.args, self.scale, self.sink)
+                     *mixed, part, count, n, y, y.stride(0), *self.args, self.scale, self.sink)
                 self.verify(y, n)
+                assert int(count.abs().max()) == 0
             return
         call("llj_gqa_prep", self.inp, self.ld, *o[:3], *rot, pos, self.seq, self.slot, self.cache, self.W, self.ldc, *mixed,
              *self.args, dt)

@@ -1662,8 +1662,9 @@ def test_gemm_grouped_dequant_equals_get_weight_bf16(hip, scale_kind):
         sc = bf16(sc)
     x = np.eye(K, dtype=np.float32)
     out = torch.empty(K, N, dtype=torch.bfloat16, device=dev)
-    call(hip, "llj_gemm_linear", 4 | (1 << 8), T(x, torch.bfloat16).data_ptr(), K, repack(hip, qw).data_ptr(),
-         sz_grouped(hip, sc, z).data_ptr(), out.data_ptr(), N, K, N, K, st())
+    # (named: a temporary's memory would be handed to the next allocation before the launch)
+    xd, wd, szd = T(x, torch.bfloat16), repack(hip, qw), sz_grouped(hip, sc, z)
+    call(hip, "llj_gemm_linear", 4 | (1 << 8), xd.data_ptr(), K, wd.data_ptr(), szd.data_ptr(), out.data_ptr(), N, K, N, K, st())
     torch.cuda.synchronize()
     wref = O.colblock_get_weight(qw, sc, z, 4, tile_cols=g, bf16=True)
     np.testing.assert_array_equal(out.float().cpu().numpy().T, wref)
